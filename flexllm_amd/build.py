@@ -1,4 +1,5 @@
 """Builds libflexllm_hip.so (gfx950) in-tree with hipcc.  `python -m flexllm_amd.build`."""
+import fcntl
 import glob
 import os
 import subprocess
@@ -22,12 +23,28 @@ def sources():
     return sorted(glob.glob(os.path.join(CSRC, "*.hip")))
 
 
-def build(verbose=False, jobs=8):
+# Parts of the library that can be built and loaded on their own (a checkout without built files then compiles what one
+# model needs and nothing else).
+COMPONENTS = {"hybrid": ("runtime", "hybrid", "gemm_float", "gemv_float", "rows_float", "latent_attn", "gla")}
+
+
+def component(name):
+    """Path of lib<flexllm>_<name>.so with the sources of COMPONENTS[name], compiled when it is missing."""
+    path = os.path.join(HERE, "libflexllm_%s.so" % name)
+    with open(os.path.join(HERE, ".build.lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)                # a second process waits for the first one's build
+        if not os.path.exists(path):
+            srcs = [os.path.join(CSRC, s + ".hip") for s in COMPONENTS[name]]
+            build(srcs=srcs, out=path, obj_dir=os.path.join(CSRC, "build", name))
+    return path
+
+
+def build(verbose=False, jobs=8, srcs=None, out=LIB, obj_dir=os.path.join(CSRC, "build")):
     objs = []
     procs = []
-    os.makedirs(os.path.join(CSRC, "build"), exist_ok=True)
-    for src in sources():
-        obj = os.path.join(CSRC, "build", os.path.basename(src)[:-4] + ".o")
+    os.makedirs(obj_dir, exist_ok=True)
+    for src in srcs or sources():
+        obj = os.path.join(obj_dir, os.path.basename(src)[:-4] + ".o")
         objs.append(obj)
         cmd = [HIPCC, *FLAGS, "-c", src, "-o", obj]
         if verbose:
@@ -36,11 +53,13 @@ def build(verbose=False, jobs=8):
         if len(procs) >= jobs:
             _drain(procs)
     _drain(procs)
-    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB, *objs]
-    out = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
-    if out.returncode != 0:
-        raise RuntimeError("link failed:\n" + out.stdout)
-    return LIB
+    part = out + ".part"                                # a reader never sees a half-written library
+    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", part, *objs]
+    res = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
+    if res.returncode != 0:
+        raise RuntimeError("link failed:\n" + res.stdout)
+    os.replace(part, out)
+    return out
 
 
 def _drain(procs):

@@ -96,31 +96,6 @@ static __global__ __launch_bounds__(256) void dec_out_quant_kernel(const int32_t
 
 static __global__ void set_state_kernel(int* state, int pos, int step) { state[0] = pos; state[1] = step; }
 
-static __global__ __launch_bounds__(64) void argmax_final_advance_kernel(const float* __restrict__ pv, const int* __restrict__ pi,
-                                                                         int nparts, int* __restrict__ token_io,
-                                                                         int* __restrict__ tokens_out, int* __restrict__ state) {
-    float best = -INFINITY;
-    int bi = 0x7fffffff;
-    for (int i = threadIdx.x; i < nparts; i += 64) {
-        const float v = pv[i];
-        const int idx = pi[i];
-        if (v > best || (v == best && idx < bi)) { best = v; bi = idx; }
-    }
-#pragma unroll
-    for (int m = 1; m < 64; m <<= 1) {
-        const float ov = __shfl_xor(best, m);
-        const int oi = __shfl_xor(bi, m);
-        if (ov > best || (ov == best && oi < bi)) { best = ov; bi = oi; }
-    }
-    if (threadIdx.x == 0) {
-        const int tok = bi == 0x7fffffff ? 0 : bi;
-        token_io[0] = tok;
-        tokens_out[state[1]] = tok;
-        state[0] += 1;
-        state[1] += 1;
-    }
-}
-
 static int dev_alloc(flexllm_llama* m, void** p, size_t bytes) {
     hipError_t e = hipMalloc(p, bytes ? bytes : 1);
     if (e != hipSuccess) {

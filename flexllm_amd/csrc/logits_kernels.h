@@ -119,6 +119,32 @@ static __global__ __launch_bounds__(64) void argmax_final_kernel(const float* __
     if (threadIdx.x == 0) result[0] = bi == 0x7fffffff ? 0 : bi;
 }
 
+// Last stage of a greedy decode step: the token goes to token_io and tokens_out[state[1]], position and step advance.
+static __global__ __launch_bounds__(64) void argmax_final_advance_kernel(const float* __restrict__ pv, const int* __restrict__ pi,
+                                                                         int nparts, int* __restrict__ token_io,
+                                                                         int* __restrict__ tokens_out, int* __restrict__ state) {
+    float best = -INFINITY;
+    int bi = 0x7fffffff;
+    for (int i = threadIdx.x; i < nparts; i += 64) {
+        const float v = pv[i];
+        const int idx = pi[i];
+        if (v > best || (v == best && idx < bi)) { best = v; bi = idx; }
+    }
+#pragma unroll
+    for (int m = 1; m < 64; m <<= 1) {
+        const float ov = __shfl_xor(best, m);
+        const int oi = __shfl_xor(bi, m);
+        if (ov > best || (ov == best && oi < bi)) { best = ov; bi = oi; }
+    }
+    if (threadIdx.x == 0) {
+        const int tok = bi == 0x7fffffff ? 0 : bi;
+        token_io[0] = tok;
+        tokens_out[state[1]] = tok;
+        state[0] += 1;
+        state[1] += 1;
+    }
+}
+
 // ---- top-k sampling (Modules/Logits.h:145-279) ------------------------------------------------------------
 // Each thread keeps the k best (value, index) of its share, ordered by value descending then index ascending; k
 // rounds of a block-wide arg-max over the threads' current heads pop the top-k in that order.  Long rows go through

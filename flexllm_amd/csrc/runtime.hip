@@ -84,6 +84,11 @@ __global__ void fill_f16_kernel(__half* dst, size_t n, uint64_t seed, float lo, 
     const size_t stride = (size_t)gridDim.x * blockDim.x;
     for (; i < n; i += stride) dst[i] = __float2half_rn(lo + width * u01(splitmix64(seed, i)));
 }
+__global__ void fill_bf16_kernel(__bf16* dst, size_t n, uint64_t seed, float lo, float width) {
+    size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    const size_t stride = (size_t)gridDim.x * blockDim.x;
+    for (; i < n; i += stride) dst[i] = (__bf16)(lo + width * u01(splitmix64(seed, i)));
+}
 }  // namespace fx
 
 using namespace fx;
@@ -192,6 +197,14 @@ int flexllm_rt_fill_uniform_f16(uint16_t* dst, size_t n, uint64_t seed, float lo
     FX_REQUIRE(dst, "fill_f16: null");
     if (n == 0) return FLEXLLM_OK;
     fill_f16_kernel<<<fill_grid(n), 256, 0, as_stream(stream)>>>((__half*)dst, n, seed, lo, hi - lo);
+    FX_LAUNCH_CHECK();
+    return FLEXLLM_OK;
+}
+
+int flexllm_rt_fill_uniform_bf16(uint16_t* dst, size_t n, uint64_t seed, float lo, float hi, void* stream) {
+    FX_REQUIRE(dst, "fill_bf16: null");
+    if (n == 0) return FLEXLLM_OK;
+    fill_bf16_kernel<<<fill_grid(n), 256, 0, as_stream(stream)>>>((__bf16*)dst, n, seed, lo, hi - lo);
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
 }

@@ -26,6 +26,7 @@ linear testbench accumulates qval * scale, Linear_Layer_Decoding_tb.cpp:171-188)
 `save_reference_parameters` writes the same files from a host weight dictionary, e.g. to hand a synthetic model to
 the reference's own testbench.
 """
+import json
 import os
 import re
 
@@ -197,3 +198,59 @@ def save_reference_parameters(param_dir, cfg, w):
         np.ascontiguousarray(w["head_w"], dtype=np.int8).tofile(os.path.join(param_dir, "lm_head.bin"))
         _write_header(os.path.join(param_dir, "w_lm_head_lm_head.h"),
                       [("w_lm_head_lm_head_s", np.asarray(w["head_s"], np.float32)), ("w_lm_head_lm_head_sum", np.asarray(w["head_sum"], np.float32))])
+
+
+# ---- safetensors ---------------------------------------------------------------------------------------------------
+_ST_TYPES = {"BF16": np.uint16, "F16": np.float16, "F32": np.float32, "I32": np.int32, "I64": np.int64, "U8": np.uint8, "I8": np.int8}
+
+
+def read_safetensors(path):
+    """{name: array} of a safetensors file: 8-byte little-endian length, that many bytes of JSON (name -> dtype, shape,
+    data_offsets), then the data.  The file is memory-mapped; bfloat16 tensors come as uint16 bit patterns."""
+    size = os.path.getsize(path)
+    if size < 8:
+        raise ParameterError("%s: not a safetensors file" % path)
+    with open(path, "rb") as f:
+        n = int.from_bytes(f.read(8), "little")
+        if n > size - 8:
+            raise ParameterError("%s: header of %d bytes in a file of %d" % (path, n, size))
+        head = json.loads(f.read(n))
+    data = np.memmap(path, np.uint8, "r") if size > 8 + n else np.zeros(8 + n, np.uint8)
+    out = {}
+    for name, t in head.items():
+        if name == "__metadata__":
+            continue
+        if t["dtype"] not in _ST_TYPES:
+            raise ParameterError("%s: %s has type %s" % (path, name, t["dtype"]))
+        dt = np.dtype(_ST_TYPES[t["dtype"]])
+        a, b = t["data_offsets"]
+        if b - a != int(np.prod(t["shape"], dtype=np.int64)) * dt.itemsize or 8 + n + b > size:
+            raise ParameterError("%s: %s does not fit its offsets" % (path, name))
+        out[name] = np.frombuffer(data[8 + n + a:8 + n + b].tobytes(), dt).reshape(t["shape"])
+    return out
+
+
+def write_safetensors(path, tensors):
+    """Writes {name: array}; uint16 arrays are stored as bfloat16 bit patterns."""
+    names = {np.dtype(v): k for k, v in _ST_TYPES.items()}
+    head, pos = {}, 0
+    arrays = {n: np.ascontiguousarray(a) for n, a in tensors.items()}
+    for n, a in arrays.items():
+        head[n] = {"dtype": names[a.dtype], "shape": list(a.shape), "data_offsets": [pos, pos + a.nbytes]}
+        pos += a.nbytes
+    text = json.dumps(head).encode()
+    text += b" " * (-len(text) % 8)
+    with open(path, "wb") as f:
+        f.write(len(text).to_bytes(8, "little") + text)
+        for a in arrays.values():
+            f.write(a.tobytes())
+
+
+def to_bf16(a):
+    """float array -> bfloat16 bit patterns (uint16), round to nearest even."""
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+    return ((u + np.uint32(0x7FFF) + ((u >> np.uint32(16)) & np.uint32(1))) >> np.uint32(16)).astype(np.uint16)
+
+
+def from_bf16(u):
+    return (np.asarray(u, np.uint16).astype(np.uint32) << np.uint32(16)).view(np.float32)

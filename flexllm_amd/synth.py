@@ -66,3 +66,10 @@ def device_uniform_f16(shape, seed, lo, hi, stream=None):
     check(lib().flexllm_rt_fill_uniform_f16(C.c_void_p(a.ptr), C.c_size_t(a.size), C.c_uint64(seed),
                                             C.c_float(lo), C.c_float(hi), _s(stream)))
     return a
+
+
+def device_uniform_bf16(shape, seed, lo, hi, stream=None):
+    a = DeviceArray(shape, np.uint16)
+    check(lib().flexllm_rt_fill_uniform_bf16(C.c_void_p(a.ptr), C.c_size_t(a.size), C.c_uint64(seed),
+                                             C.c_float(lo), C.c_float(hi), _s(stream)))
+    return a

@@ -493,6 +493,84 @@ int flexllm_hmt_retrieve(const float* q, const float* kmem, const float* mmem, f
 int flexllm_hmt_stage_input(const float* emb, const float* t_embed, const float* p_buf, float* x_out, int stage, int seq_off,
                             int cur_len, int cur_sum_len, int rec_len, int tail_p, int rows, int hidden, void* stream);
 
+/* ---- floating-point decoder models: layers of latent attention and gated linear attention -------------------------
+ * A decoder whose layers are chosen one by one (no counterpart in the reference, which has one quantised graph): each
+ * layer is a mixer and a feed-forward, both with an RMS norm before and after (weights stored around zero:
+ * rms(x) * (1 + w)) and a float32 residual.  dtype 0: weights, activations between kernels and cached rows in bfloat16
+ * with float32 sums; dtype 1: everything in float32.  Norms, scores and softmax, routers, the residual and every state
+ * are float32 in both.  Weight pointers are device bfloat16 arrays, row-major [out][in], copied and repacked by create.
+ *
+ * Mixers
+ *   FLEXLLM_MIX_LATENT  latent attention: W_dkv h = [latent | shared key part]; the normed latent and the rotated key part
+ *                       are cached (one row per token); keys W_uk c and values W_uv c per head.  window > 0: the last
+ *                       `window` positions are seen, 0: all.  kv_from >= 0: the layer reads the rows of that earlier
+ *                       layer and has no dkv of its own.  Rotation: neighbouring pairs, base rot_base, with yarn != 0
+ *                       the frequencies are interpolated between f and f / yarn_factor.
+ *   FLEXLLM_MIX_GLA     gated linear attention, decay per key channel sigmoid(W_a2 W_a1 h + b)^(1/tau), float32 state
+ * Feed-forwards
+ *   FLEXLLM_FF_NONE, FLEXLLM_FF_DENSE (clamped gated unit g sigmoid(1.702 g)(u + 1), g = min(gate, limit),
+ *   u = clamp(up, -limit, limit)), FLEXLLM_FF_MOE (`top` of `experts` by softmax, weights divided by their sum; an
+ *   optional shared expert times sigmoid(W_sg h))
+ *
+ * Sequences live in slots: a slot holds the cached rows, the states and the length of one sequence.  reset starts it
+ * afresh (nothing of the previous sequence is read again).  One object is used from one stream at a time. */
+#define FLEXLLM_MIX_LATENT 0
+#define FLEXLLM_MIX_GLA 1
+#define FLEXLLM_FF_NONE 0
+#define FLEXLLM_FF_DENSE 1
+#define FLEXLLM_FF_MOE 2
+typedef struct {
+    int layers, width, vocab, max_pos, slots, dtype;
+    float eps;
+} flexllm_hybrid_config;
+typedef struct {
+    int mixer, heads, dim, vdim;
+    int rot_dim, kv_rank, window, kv_from;      /* latent attention */
+    int yarn;
+    float scale;
+    double rot_base, yarn_factor, yarn_original, yarn_fast, yarn_slow;
+    int a_rank;                                 /* gated linear attention */
+    float tau;
+    int ff_kind, ff, experts, top, shared_ff;   /* ff: of the dense layer or of an expert; shared_ff 0: none */
+    float limit, shared_limit;
+} flexllm_hybrid_layer;
+typedef struct {
+    const uint16_t *norm1, *norm1b, *norm2, *norm2b;                       /* [width] */
+    const uint16_t *q, *o;                                                 /* both mixers */
+    const uint16_t *dkv, *dkv_norm, *uk, *uv;                              /* latent attention */
+    const uint16_t *k, *v, *g, *a1, *a2, *a2_bias, *head_norm;             /* gated linear attention */
+    const uint16_t *gate, *up, *down;                                      /* dense */
+    const uint16_t *router, *shared_gate, *shared_up, *shared_down, *shared_sg;
+    const uint16_t *const *expert_gate, *const *expert_up, *const *expert_down;   /* host arrays of `experts` device pointers */
+} flexllm_hybrid_layer_weights;
+typedef struct {
+    const uint16_t *embed, *final_norm, *head;
+} flexllm_hybrid_weights;
+
+typedef struct flexllm_hybrid flexllm_hybrid;
+int flexllm_hybrid_create(flexllm_hybrid** out, const flexllm_hybrid_config* cfg, const flexllm_hybrid_layer* layers,
+                          const flexllm_hybrid_weights* w, const flexllm_hybrid_layer_weights* lw);
+int flexllm_hybrid_destroy(flexllm_hybrid* m);
+int flexllm_hybrid_reset(flexllm_hybrid* m, int slot, void* stream);
+/* Tokens the slot holds. */
+int flexllm_hybrid_length(const flexllm_hybrid* m, int slot, int* length);
+/* Run n further tokens (device ids) of the slot's sequence from what its cache and states hold.  want (host, ascending
+ * places in 0..n-1) names the n_want tokens whose logits are written to logits (device [n_want][vocab]).  layers_out
+ * (device [layers][n][width] or NULL) receives the residual after every layer. */
+int flexllm_hybrid_step(flexllm_hybrid* m, int slot, const int* tokens, int n, const int* want, int n_want, float* logits,
+                        float* layers_out, void* stream);
+/* `steps` tokens from *token_io (device; fed first, the last drawn token on return) into tokens_out (device [steps]):
+ * the largest logit, or with top_k > 0 a draw from the top_k largest with rands[step] (device).  use_graph: one step is
+ * captured in a HIP graph and replayed (needs a stream of its own). */
+int flexllm_hybrid_decode(flexllm_hybrid* m, int slot, int* token_io, int steps, const float* rands, int top_k, int* tokens_out,
+                          int use_graph, void* stream);
+/* Prompt to tokens in one slot: all prompt tokens but the last in one go, then the decode loop from the last one. */
+int flexllm_hybrid_generate(flexllm_hybrid* m, int slot, const int* prompt, int n_prompt, int steps, const float* rands, int top_k,
+                            int* tokens_out, int use_graph, void* stream);
+/* Synchronises and reports a token id outside the vocabulary (FLEXLLM_EINVAL; id 0 was used). */
+int flexllm_hybrid_check(flexllm_hybrid* m);
+int flexllm_rt_fill_uniform_bf16(uint16_t* dst, size_t n, uint64_t seed, float lo, float hi, void* stream);
+
 #ifdef __cplusplus
 }
 #endif
