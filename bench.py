@@ -326,6 +326,126 @@ def module_legs(fx, lib, synth, ops, stream, Event, peaks=None):
     return out
 
 
+# ---- Nifunex: layers of real models' sizes, random weights ------------------------------------------------------------
+BF16_PEAK_TFLOPS = 2500.0      # MI355X published dense bf16 MFMA rate
+
+
+def nifunex_config(name):
+    """Sizes for --nifunex.  1b-dense has the hidden size, feed-forward, layer count and vocabulary of Llama-3.2-1B, the
+    framework's other model; 1b-moe and 8b-dense take their feed-forwards from published mixtures and 8B models."""
+    heads, width, layers, vocab = {"1b-dense": (16, 2048, 16, 128256), "1b-moe": (16, 2048, 8, 128256), "8b-dense": (32, 4096, 4, 128256)}[name]
+    mlp = {"1b-dense": {"kind": "dense", "ff": 8192, "limit": 7.0}, "8b-dense": {"kind": "dense", "ff": 14336, "limit": 7.0},
+           "1b-moe": {"kind": "moe", "router": {"experts": 64, "top": 6}, "expert": {"ff": 1024, "limit": 7.0}, "shared": {"ff": 2048, "limit": 7.0}}}[name]
+    rot = {"base": 10000.0, "dims": 64, "scaling": {"factor": 40.0, "original": 4096, "fast": 32.0, "slow": 1.0}}
+    out = []
+    for i in range(layers):
+        if i % 2 == 0:
+            mx = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5, "mask": {"size": 1024}, "rot": rot}
+            if i % 4 == 2:
+                mx["kv_from"] = i - 2
+            out.append({"type": "latent_attention", "mixer": mx, "mlp": mlp})
+        else:
+            out.append({"type": "gla", "mixer": {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0}, "mlp": mlp})
+    return {"architecture": "Nifunex", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "layers": out}
+
+
+def nifunex_work(cfg, shapes, tokens, context):
+    """(bytes that one decoded token reads at `context`, operations of a prompt of `tokens`: multiply-adds counted twice,
+    attention over the visible pairs only, the recurrence in its token-by-token form)."""
+    size = lambda n: int(np.prod(shapes[n]))
+    per_token, by, ops = 0, 0, 0
+    for i, ly in enumerate(cfg["layers"]):
+        mx, mlp = ly["mixer"], ly["mlp"]
+        names = [n for n in shapes if n.startswith("l%d." % i) and len(shapes[n]) == 2]
+        mats = sum(size(n) for n in names if ".mlp.e" not in n)
+        if mlp["kind"] == "moe":
+            mats += mlp["router"]["top"] * 3 * cfg["width"] * mlp["expert"]["ff"]
+        by += 2 * mats
+        if ly["type"] == "gla":
+            state = mx["heads"] * mx["dim"] * mx["vdim"]
+            by += 8 * state
+            ops += 2 * tokens * mats + 4 * tokens * state
+        else:
+            uk_uv = size("l%d.mix.uk" % i) + size("l%d.mix.uv" % i)
+            win = (mx.get("mask") or {}).get("size") or context
+            by += 2 * min(win, context) * (mx["kv_rank"] + mx["rot_dim"])
+            pairs = sum(min(p + 1, win) for p in range(tokens))
+            ops += 2 * tokens * mats + 2 * pairs * mx["heads"] * (mx["dim"] + mx["rot_dim"] + mx["vdim"])
+    return by + 2 * size("head"), ops
+
+
+def nifunex_leg(name, steps, warmup, prompts=(1024, 4096), seed=3):
+    import flexllm_amd as fx
+    from flexllm_amd import synth
+    from flexllm_amd.device import Event, device_sync
+    from flexllm_amd.nifunex import Nifunex, tensor_shapes
+    cfg = nifunex_config(name)
+    shapes = tensor_shapes(cfg)
+    m = Nifunex.synthetic(cfg, seed=seed, max_pos=max(prompts) + warmup + steps + 8)
+    st = m.stream()
+    toks = fx.to_device(np.random.default_rng(7).integers(0, cfg["vocab"], max(prompts)).astype(np.int32))
+    out = {"config": {"width": cfg["width"], "layers": len(cfg["layers"]), "vocab": cfg["vocab"], "mlp": cfg["layers"][0]["mlp"]}, "prefill": {}}
+
+    def prompt(n):
+        slot = m.pool.acquire("p")
+        fx.check(fx.lib().flexllm_hybrid_step(m.handle, slot, C.c_void_p(toks.ptr), n, None, 0, None, None, st.handle))
+        m.pool.release("p")
+
+    for n in prompts:
+        us = _time(st, Event, lambda i: prompt(n), 5)
+        _, ops = nifunex_work(cfg, shapes, n, n)
+        out["prefill"][str(n)] = {"ms": round(us / 1e3, 3), "tokens_per_s": round(n / us * 1e6, 1), "TFLOPs": round(ops / us / 1e6, 1),
+                                  "mfma_frac": round(ops / us / 1e6 / BF16_PEAK_TFLOPS, 4)}
+    slot = m.pool.acquire("d")
+    fx.check(fx.lib().flexllm_hybrid_step(m.handle, slot, C.c_void_p(toks.ptr), max(prompts), None, 0, None, None, st.handle))
+    io, gen = fx.to_device(np.array([17], np.int32)), fx.zeros((max(steps, warmup, 1),), np.int32)
+    if warmup:
+        m.decode(slot, io, warmup, gen)
+    st.sync()
+    e0, e1 = Event(), Event()
+    e0.record(st)
+    m.decode(slot, io, steps, gen)
+    e1.record(st)
+    e1.sync()
+    device_sync()
+    m.check()
+    us = e0.elapsed_ms(e1) * 1e3 / steps
+    by, _ = nifunex_work(cfg, shapes, 1, max(prompts))
+    out["decode"] = {"context": max(prompts), "us_per_token": round(us, 2), "tokens_per_s": round(1e6 / us, 1), "bytes_per_token": by,
+                     "GBs": round(by / us / 1e3, 1), "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4), "distinct_tokens": len(set(gen.numpy()[:steps].tolist()))}
+    m.close()
+    return out
+
+
+def nifunex_main(args):
+    """--nifunex: decode and prefill of the Nifunex sizes beside Llama-3.2-1B W8A8 in the same process.  One JSON line."""
+    import flexllm_amd as fx
+    from flexllm_amd import llama, synth
+    from flexllm_amd.device import Event
+    res = {"metric": "Nifunex decode tok/s + prefill ms", "dtype": "bf16", "data": "synthetic", "device": fx.device.device_name(), "sizes": {}}
+    for name in args.nifunex.split(","):
+        res["sizes"][name] = nifunex_leg(name, args.steps, args.warmup)
+    if not args.no_prefill:
+        cfg = llama.make_config()
+        model = llama.Llama(cfg, llama.synth_weights(cfg, seed=1, device=True, embed_range=0.03))
+        st = fx.Stream()
+        tok, out = fx.to_device(np.array([12345], np.int32)), fx.zeros((args.steps,), np.int32)
+        us = _time(st, Event, lambda i: model.decode_greedy(tok, cfg["max_pos"] - args.steps, args.steps, out, use_graph=False, stream=st), 2) / args.steps
+        by = bytes_per_token(cfg, cfg["max_pos"] - args.steps / 2.0)
+        leg = {"decode": {"context": cfg["max_pos"], "us_per_token": round(us, 2), "tokens_per_s": round(1e6 / us, 1), "GBs": round(by / us / 1e3, 1),
+                          "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4)}, "prefill": {}}
+        for n in (1024, 4096):
+            x = synth.device_uniform_f32((n, cfg["hidden"]), 4243, -1.7, 1.7)
+            us = _time(st, Event, lambda i: model.prefill_hidden(x, stream=st), 3)
+            H, I = cfg["hidden"], cfg["inter"]
+            ops = cfg["layers"] * (2 * n * (H * (H + 2 * cfg["kv_hidden"]) + H * H + 3 * I * H) + 2 * n * (n + 1) * H)
+            leg["prefill"][str(n)] = {"ms": round(us / 1e3, 3), "tokens_per_s": round(n / us * 1e6, 1), "TOPs": round(ops / us / 1e6, 1),
+                                      "mfma_frac": round(ops / us / 1e6 / INT8_PEAK_TOPS, 4)}
+        model.close()
+        res["llama_3.2_1b_w8a8"] = leg
+    print(json.dumps(res))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -345,6 +465,9 @@ def main():
     ap.add_argument("--module-probe", action="store_true",
                     help="only run the single-module legs (decode linear, Hadamard + quantisation, prefill linear stack, "
                          "prefill attention, W4A4 linears) and exit: the short command the per-kernel counter runs use")
+    ap.add_argument("--nifunex", nargs="?", const="1b-dense,1b-moe,8b-dense", default=None, metavar="SIZES",
+                    help="only run the Nifunex sizes (1b-dense, 1b-moe, 8b-dense; all when none is named) and, unless --no-prefill, "
+                         "Llama-3.2-1B W8A8 beside them")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on one GPU only (no collectives, no sharding); use --gpus 1", file=sys.stderr)
@@ -355,6 +478,9 @@ def main():
     from flexllm_amd.device import Event, device_sync
 
     lib = fx.lib()
+    if args.nifunex:
+        nifunex_main(args)
+        return
     if args.copy_probe:
         n = 1 << 30
         src = synth.device_i8((n,), 1)
