@@ -94,18 +94,20 @@ struct LatentDims {
     float scale, eps;
     int capacity;
 };
-// Rows of the q / dkv projection: q [tokens][ldq] of QT (float in the one-token path), raw [tokens][ld_raw] float32
-// (null: the layer has no rows of its own).
-template <typename ET> int latent_store(const LatentDims& d, void* q, int ldq, int q_f32, const float* raw, int ld_raw,
-                                        const float* norm_w, const float* cos_t, const float* sin_t, ET* cache, const int* state,
-                                        int tokens, hipStream_t st);
+// Rows of the q / dkv projection: rotates the queries' rotated part in q [tokens][ldq] and leaves the tokens' own rows in
+// the cache (raw [tokens][ld_raw] float32; null: the layer has no rows of its own).
+template <typename ET> int latent_store(const LatentDims& d, ET* q, int ldq, const float* raw, int ld_raw, const float* norm_w, const float* cos_t,
+                                        const float* sin_t, ET* cache, const int* state, int tokens, hipStream_t st);
 // Attention over the stored rows themselves: the unrotated query is carried into the latent space through W_uk, the
-// context back through W_uv.  Any size; for few tokens.  q: float32 or ET with the rotated part already rotated.
-// Scratch: latent_absorbed_scratch floats per token.  o: [tokens][ldo], float32 or ET.
+// context back through W_uv.  Any size; for few tokens.  q as latent_store leaves it.  Scratch:
+// latent_absorbed_scratch floats per token.
 size_t latent_absorbed_scratch(const LatentDims& d);
-template <typename ET> int latent_absorbed(const LatentDims& d, const void* q, int ldq, int q_f32, const ET* w_uk, const ET* w_uv,
-                                           const ET* cache, const int* state, int tok0, int tokens, float* scratch, void* o, int ldo,
-                                           int o_f32, hipStream_t st);
+template <typename ET> int latent_absorbed(const LatentDims& d, const ET* q, int ldq, const ET* w_uk, const ET* w_uv, const ET* cache,
+                                           const int* state, int tok0, int tokens, float* scratch, ET* o, int ldo, hipStream_t st);
+// Both in the one-token path: q, raw and o float32, q not rotated yet and left alone.
+template <typename ET> int latent_decode(const LatentDims& d, const float* q, int ldq, const float* raw, int ld_raw, const float* norm_w,
+                                         const float* cos_t, const float* sin_t, const ET* w_uk, const ET* w_uv, ET* cache, const int* state,
+                                         int tokens, float* scratch, float* o, int ldo, hipStream_t st);
 // Attention of many tokens with keys and values formed once: k [rows][ldk] (heads x dim), vt [heads x vdim][ldv] for the
 // stored rows kv0 .. kv0+rows-1.  bfloat16 only.
 bool latent_flash_ok(const LatentDims& d);

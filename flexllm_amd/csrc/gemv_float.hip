@@ -1,8 +1,8 @@
 // Linears of one token: y = W h with W of ET (bfloat16 or float32) streamed once, h float32 in LDS.
 //
-// A workgroup of 256 threads owns R weight rows; thread t reads 16-byte pieces t, t + 256, ... of each.  The first
-// R x S pieces are requested before the prologue (residual, norms, expert choice) runs, so that its latency lies under
-// the weight stream.  The R sums are reduced together (multi_sum_step).
+// A workgroup of 256 threads walks groups of R weight rows; thread t reads 16-byte pieces t, t + 256, ... of each row.
+// The first two groups are requested before the prologue (residual, norms) runs, so that its latency lies under the weight
+// stream, and two groups stay in flight after that.  The R sums are reduced together (multi_sum_step).
 #include "float_ops.h"
 
 namespace fx {
@@ -34,22 +34,22 @@ __device__ __forceinline__ void route_wave(const float* __restrict__ z, int expe
     float sum = 0.0f;
     for (int k = 0; k < top; k++) {
         float best = -2.0f;
-        int bi = 0x7fffffff;
 #pragma unroll
         for (int i = 0; i < kMaxExperts / 64; i++) {
             if (i * 64 >= experts) break;
-            if (v[i] > best) { best = v[i]; bi = i * 64 + lane; }
+            best = fmaxf(best, v[i]);
         }
-#pragma unroll
-        for (int m = 1; m < 64; m <<= 1) {
-            const float ov = __shfl_xor(best, m);
-            const int oi = __shfl_xor(bi, m);
-            if (ov > best || (ov == best && oi < bi)) { best = ov; bi = oi; }
-        }
+        best = wave_max(best);
+        int bi = -1;                                      // lowest index that holds the maximum
 #pragma unroll
         for (int i = 0; i < kMaxExperts / 64; i++) {
             if (i * 64 >= experts) break;
-            if (i * 64 + lane == bi) v[i] = -1.0f;
+            const unsigned long long hit = __ballot(v[i] == best);
+            if (bi < 0 && hit) {
+                const int l = __builtin_ctzll(hit);
+                bi = i * 64 + l;
+                if (lane == l) v[i] = -1.0f;
+            }
         }
         const float s = best / den;
         sum += s;
@@ -59,17 +59,39 @@ __device__ __forceinline__ void route_wave(const float* __restrict__ z, int expe
         for (int k = 0; k < top; k++) wt[k] = wt[k] / (sum + 1e-20f);
 }
 
-template <typename ET, int R, int S, int PRO>
+// VQ: the norm prologue keeps its vectors in registers, VQ float4 per thread (k a multiple of 4, at most 1024 VQ); 0: any k,
+// through LDS.  Only used with PRO = 1.
+template <typename ET, int R, int S, int PRO, int VQ>
 __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     constexpr int CE = Chunk<ET>::N;
-    extern __shared__ __attribute__((aligned(16))) float xs[];     // [kpad] the vector, then the reduction area
-    __shared__ float red[4 * (R > 4 ? R : 4)];
+    extern __shared__ __attribute__((aligned(16))) float xs[];     // [kpad] the vector
+    __shared__ float red[2][4 * R];
+    __shared__ float nred[4];
     __shared__ int sel[kMaxTop];
     __shared__ float wt[kMaxTop];
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
     const int tok = PRO == 2 ? blockIdx.y / g.top : blockIdx.y;
-    const int row0 = blockIdx.x * R;
     const ET* w = static_cast<const ET*>(g.w);
+    const float* x = g.x + (size_t)tok * g.ldx;
+    // ---- requests for the vector go out first: loads return in order, and the weights behind them are a long stream
+    constexpr int Q = VQ > 0 ? VQ : 1;
+    f32x4 xv[Q], yv[Q], gb[Q], gv[Q];
+    const int k4 = g.k >> 2;
+    const bool have_y = PRO == 1 && g.y != nullptr;
+    if constexpr (PRO == 1 && VQ > 0) {
+        const f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
+        const float* y = g.y + (size_t)tok * g.ldy;
+#pragma unroll
+        for (int i = 0; i < Q; i++) {
+            const int c = t + 256 * i;
+            const bool in = c < k4;
+            yv[i] = in && have_y ? *reinterpret_cast<const f32x4*>(y + 4 * c) : zero;
+            xv[i] = in ? *reinterpret_cast<const f32x4*>(x + 4 * c) : zero;
+            gb[i] = in && have_y ? *reinterpret_cast<const f32x4*>(g.gb + 4 * c) : zero;
+            gv[i] = in ? *reinterpret_cast<const f32x4*>(g.g + 4 * c) : zero;
+        }
+        __builtin_amdgcn_sched_barrier(0);
+    }
     if constexpr (PRO == 2) {
         if (wave == 0) route_wave(g.route + (size_t)tok * g.ld_route, g.experts, g.top, sel, wt);
         __syncthreads();
@@ -78,34 +100,71 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
         if (blockIdx.x == 0 && t == 0) { g.pick[blockIdx.y] = sel[slot]; g.pick_w[blockIdx.y] = wt[slot]; }
     }
     const int nchunk = g.kpad / CE;                       // 16-byte pieces of a row
-    uint4 pre[R][S];
+    const int ng = (g.n + R - 1) / R, G = gridDim.x;      // groups of R rows, dealt to the workgroups in turn
+    i32x4 buf[2][R][S];
+    auto piece = [&](int row, int c) { return *reinterpret_cast<const i32x4*>(w + (size_t)min(row, g.n - 1) * g.kpad + c * CE); };
+    auto load = [&](int b, int grp) {
 #pragma unroll
-    for (int r = 0; r < R; r++)
+        for (int r = 0; r < R; r++)
 #pragma unroll
-        for (int s = 0; s < S; s++) {
-            const int c = s * 256 + t;
-            pre[r][s] = c < nchunk ? *reinterpret_cast<const uint4*>(w + (size_t)min(row0 + r, g.n - 1) * g.kpad + c * CE)
-                                   : make_uint4(0, 0, 0, 0);
-        }
+            for (int s = 0; s < S; s++) {
+                const int c = s * 256 + t;
+                buf[b][r][s] = c < nchunk ? piece(grp * R + r, c) : i32x4{0, 0, 0, 0};
+            }
+    };
+    const int g0 = blockIdx.x;
+    load(0, g0);
+    if (g0 + G < ng) load(1, g0 + G);
+    __builtin_amdgcn_sched_barrier(0);
     // ---- the vector
-    const float* x = g.x + (size_t)tok * g.ldx;
-    if constexpr (PRO == 1) {
+    if constexpr (PRO == 1 && VQ > 0) {
         float rs = 0.0f;
-        if (g.y) {
+        if (have_y) {
+            float ss = 0.0f;
+#pragma unroll
+            for (int i = 0; i < Q; i++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) ss = fma_f(yv[i][e], yv[i][e], ss);
+            rs = 1.0f / sqrtf(block_sum<4>(ss, nred) / (float)g.k + g.eps);
+        }
+        float ss = 0.0f;
+#pragma unroll
+        for (int i = 0; i < Q; i++)
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                if (have_y) xv[i][e] = xv[i][e] + yv[i][e] * rs * gb[i][e];
+                ss = fma_f(xv[i][e], xv[i][e], ss);
+            }
+        const float rx = 1.0f / sqrtf(block_sum<4>(ss, nred) / (float)g.k + g.eps);
+#pragma unroll
+        for (int i = 0; i < Q; i++) {
+            const int c = t + 256 * i;
+            f32x4 h;
+#pragma unroll
+            for (int e = 0; e < 4; e++) h[e] = xv[i][e] * rx * gv[i][e];
+            if (4 * c < g.kpad) *reinterpret_cast<f32x4*>(xs + 4 * c) = h;
+            if (blockIdx.x == 0 && c < k4) {
+                if (g.x_new) *reinterpret_cast<f32x4*>(g.x_new + (size_t)tok * g.ldx + 4 * c) = xv[i];
+                if (g.h_out) *reinterpret_cast<f32x4*>(g.h_out + (size_t)tok * g.ldh + 4 * c) = h;
+            }
+        }
+    } else if constexpr (PRO == 1) {
+        float rs = 0.0f;
+        if (have_y) {
             const float* y = g.y + (size_t)tok * g.ldy;
             float ss = 0.0f;
             for (int i = t; i < g.k; i += 256) { const float v = y[i]; xs[i] = v; ss = fma_f(v, v, ss); }
-            rs = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)g.k + g.eps);
+            rs = 1.0f / sqrtf(block_sum<4>(ss, nred) / (float)g.k + g.eps);
         }
         float ss = 0.0f;
         for (int i = t; i < g.k; i += 256) {
             float v = x[i];
-            if (g.y) v = v + xs[i] * rs * g.gb[i];
+            if (have_y) v = v + xs[i] * rs * g.gb[i];
             xs[i] = v;
             ss = fma_f(v, v, ss);
             if (blockIdx.x == 0 && g.x_new) g.x_new[(size_t)tok * g.ldx + i] = v;
         }
-        const float rx = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)g.k + g.eps);
+        const float rx = 1.0f / sqrtf(block_sum<4>(ss, nred) / (float)g.k + g.eps);
         for (int i = t; i < g.kpad; i += 256) {
             const float v = i < g.k ? xs[i] * rx * g.g[i] : 0.0f;
             xs[i] = v;
@@ -116,68 +175,72 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     }
     __syncthreads();
     // ---- the products
-    float acc[R];
-#pragma unroll
-    for (int r = 0; r < R; r++) acc[r] = 0.0f;
-    auto dot = [&](int c, const uint4 (&u)[R]) {
-        float xv[CE];
+    auto dot = [&](int c, const i32x4& u, float& acc) {
+        float wv[CE];
+        Chunk<ET>::unpack(make_uint4(u[0], u[1], u[2], u[3]), wv);
 #pragma unroll
         for (int q = 0; q < CE / 4; q++) {
             const f32x4 v = *reinterpret_cast<const f32x4*>(xs + c * CE + q * 4);
 #pragma unroll
-            for (int e = 0; e < 4; e++) xv[q * 4 + e] = v[e];
-        }
-#pragma unroll
-        for (int r = 0; r < R; r++) {
-            float wv[CE];
-            Chunk<ET>::unpack(u[r], wv);
-#pragma unroll
-            for (int e = 0; e < CE; e++) acc[r] = fma_f(wv[e], xv[e], acc[r]);
+            for (int e = 0; e < 4; e++) acc = fma_f(wv[q * 4 + e], v[e], acc);
         }
     };
+    auto process = [&](int b, int grp) {
+        float acc[R];
 #pragma unroll
-    for (int s = 0; s < S; s++) {
-        const int c = s * 256 + t;
-        if (c < nchunk) {
-            uint4 u[R];
+        for (int r = 0; r < R; r++) acc[r] = 0.0f;
 #pragma unroll
-            for (int r = 0; r < R; r++) u[r] = pre[r][s];
-            dot(c, u);
+        for (int s = 0; s < S; s++) {
+            const int c = min(s * 256 + t, nchunk - 1);   // pieces beyond the row were filled with zeros
+#pragma unroll
+            for (int r = 0; r < R; r++) dot(c, buf[b][r][s], acc[r]);
         }
-    }
-    for (int c = S * 256 + t; c < nchunk; c += 256) {
-        uint4 u[R];
+        for (int c = S * 256 + t; c < nchunk; c += 256)
 #pragma unroll
-        for (int r = 0; r < R; r++) u[r] = *reinterpret_cast<const uint4*>(w + (size_t)min(row0 + r, g.n - 1) * g.kpad + c * CE);
-        dot(c, u);
-    }
-    multi_sum_step<R, 1>(acc, lane);
-    if (lane < R) red[wave * R + multi_row<R>(lane)] = acc[0];
-    __syncthreads();
-    if (t < R) {
-        const int row = row0 + t;
-        float v[2];
+            for (int r = 0; r < R; r++) dot(c, piece(grp * R + r, c), acc[r]);
+        multi_sum_step<R, 1>(acc, lane);
+        if (lane < R) red[b][wave * R + multi_row<R>(lane)] = acc[0];
+        __syncthreads();                                  // red alternates with the buffer: one barrier per group is enough
+        if (t < R) {
+            const int row = grp * R + t;
+            float v[2];
 #pragma unroll
-        for (int i = 0; i < 2; i++) {
-            const int r = i == 0 ? t : min(t + 1, R - 1);
-            v[i] = (red[r] + red[R + r]) + (red[2 * R + r] + red[3 * R + r]);
+            for (int i = 0; i < 2; i++) {
+                const int r = min(t + i, R - 1);
+                v[i] = (red[b][r] + red[b][R + r]) + (red[b][2 * R + r] + red[b][3 * R + r]);
+            }
+            if (row < g.n) {
+                const size_t o = blockIdx.y;
+                if (row >= g.n_split) g.out32[o * g.ldo32 + row - g.n_split] = v[0];
+                else if (!g.glu) g.out[o * g.ldo + row] = v[0];
+                else if ((row & 1) == 0) g.out[o * g.ldo + (row >> 1)] = clamped_glu_f(v[0], v[1], g.limit);
+            }
         }
-        if (row < g.n) {
-            const size_t o = blockIdx.y;
-            if (row >= g.n_split) g.out32[o * g.ldo32 + row - g.n_split] = v[0];
-            else if (!g.glu) g.out[o * g.ldo + row] = v[0];
-            else if ((row & 1) == 0) g.out[o * g.ldo + (row >> 1)] = clamped_glu_f(v[0], v[1], g.limit);
+    };
+    for (int grp = g0; grp < ng; grp += 2 * G) {
+        process(0, grp);
+        if (grp + 2 * G < ng) load(0, grp + 2 * G);
+        if (grp + G < ng) {
+            process(1, grp + G);
+            if (grp + 3 * G < ng) load(1, grp + 3 * G);
         }
     }
 }
 
 template <typename ET, int R, int S>
 static int launch_gemv_rs(const GemvArgs& g, int pro, int rows_y, hipStream_t st) {
-    const dim3 grid((g.n + R - 1) / R, rows_y);
+    // workgroups that share the chip at a time; each walks its groups with the next one's weights in flight
+    int wgs = 1024 / rows_y;
+    if (wgs < 128) wgs = 128;
+    const int ng = (g.n + R - 1) / R;
+    const dim3 grid(ng < wgs ? ng : wgs, rows_y);
     const size_t lds = (size_t)g.kpad * sizeof(float);
-    if (pro == 0) gemv_float_kernel<ET, R, S, 0><<<grid, 256, lds, st>>>(g);
-    else if (pro == 1) gemv_float_kernel<ET, R, S, 1><<<grid, 256, lds, st>>>(g);
-    else gemv_float_kernel<ET, R, S, 2><<<grid, 256, lds, st>>>(g);
+    const bool vec = g.k % 4 == 0 && g.ldx % 4 == 0 && g.ldy % 4 == 0 && g.ldh % 4 == 0;
+    if (pro == 0) gemv_float_kernel<ET, R, S, 0, 0><<<grid, 256, lds, st>>>(g);
+    else if (pro == 2) gemv_float_kernel<ET, R, S, 2, 0><<<grid, 256, lds, st>>>(g);
+    else if (vec && g.kpad <= 2048) gemv_float_kernel<ET, R, S, 1, 2><<<grid, 256, lds, st>>>(g);
+    else if (vec && g.kpad <= 4096) gemv_float_kernel<ET, R, S, 1, 4><<<grid, 256, lds, st>>>(g);
+    else gemv_float_kernel<ET, R, S, 1, 0><<<grid, 256, lds, st>>>(g);
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
 }
@@ -190,17 +253,12 @@ int gemv_float(const GemvArgs& g, int pro, int tokens, hipStream_t st) {
                "gemv_float: %d experts, top %d (at most %d, %d)", g.experts, g.top, kMaxExperts, kMaxTop);
     const int per = 256 * Chunk<ET>::N, steps = (g.kpad + per - 1) / per;
     const int rows_y = pro == 2 ? tokens * g.top : tokens;
-    auto wgs = [&](int r) { return (g.n + r - 1) / r * rows_y; };
     if (steps == 1) {
-        if (wgs(16) >= 512) return launch_gemv_rs<ET, 16, 1>(g, pro, rows_y, st);
-        if (wgs(8) >= 384) return launch_gemv_rs<ET, 8, 1>(g, pro, rows_y, st);
+        if ((g.n + 7) / 8 * rows_y >= 512) return launch_gemv_rs<ET, 8, 1>(g, pro, rows_y, st);
         return launch_gemv_rs<ET, 4, 1>(g, pro, rows_y, st);
     }
-    if (steps == 2) {
-        if (wgs(8) >= 384) return launch_gemv_rs<ET, 8, 2>(g, pro, rows_y, st);
-        return launch_gemv_rs<ET, 4, 2>(g, pro, rows_y, st);
-    }
-    return launch_gemv_rs<ET, 4, 4>(g, pro, rows_y, st);
+    if (steps == 2) return launch_gemv_rs<ET, 4, 2>(g, pro, rows_y, st);
+    return launch_gemv_rs<ET, 2, 4>(g, pro, rows_y, st);
 }
 template int gemv_float<bf16_t>(const GemvArgs&, int, int, hipStream_t);
 template int gemv_float<float>(const GemvArgs&, int, int, hipStream_t);
@@ -260,63 +318,67 @@ template int moe_down_small<float>(const MoeDownArgs&, int, hipStream_t);
 static __global__ __launch_bounds__(256) void moe_clear_kernel(int* counts, int n) {
     for (int i = threadIdx.x; i < n; i += 256) counts[i] = 0;
 }
-static __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ route, int ld, int rows, int experts, int top,
-                                                               int* __restrict__ pick, float* __restrict__ pick_w, int* __restrict__ counts) {
-    __shared__ int sel[4][kMaxTop];
-    __shared__ float wt[4][kMaxTop];
-    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, row = blockIdx.x * 4 + wave;
-    if (row >= rows) return;
-    route_wave(route + (size_t)row * ld, experts, top, sel[wave], wt[wave]);
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-    if (lane < top) {
-        const int e = sel[wave][lane];
-        pick[row * top + lane] = e;
-        pick_w[row * top + lane] = wt[wave][lane];
-        atomicAdd(&counts[e], 1);
-    }
-}
-// Place every (row, choice) in its expert's run; block 0 also cuts the runs into tiles.
-static __global__ __launch_bounds__(256) void moe_place_kernel(int rows, int experts, int top, int tile_rows, const int* __restrict__ pick,
-                                                               int* __restrict__ counts, int* __restrict__ pos_of, int* __restrict__ row_src,
-                                                               int4* __restrict__ tiles, int* __restrict__ n_tiles) {
-    __shared__ int first[kMaxExperts + 1], tile0[kMaxExperts + 1];
-    __shared__ int part[256], part_t[256];
-    const int t = threadIdx.x;
-    const int per = (experts + 255) / 256;
-    int s = 0, st = 0;
-    for (int i = 0; i < per; i++) {
-        const int e = t * per + i;
-        if (e < experts) { s += counts[e]; st += (counts[e] + tile_rows - 1) / tile_rows; }
-    }
-    part[t] = s; part_t[t] = st;
+constexpr int kPlanT = 1024, kRouteRows = 64;              // rows per workgroup of the route kernel
+static __global__ __launch_bounds__(kPlanT) void moe_route_kernel(const float* __restrict__ route, int ld, int rows, int experts, int top,
+                                                                  int* __restrict__ pick, float* __restrict__ pick_w, int* __restrict__ counts) {
+    __shared__ int sel[kPlanT / 64][kMaxTop], hist[kMaxExperts];
+    __shared__ float wt[kPlanT / 64][kMaxTop];
+    const int t = threadIdx.x, wave = t >> 6, lane = t & 63;
+    for (int e = t; e < experts; e += kPlanT) hist[e] = 0;
     __syncthreads();
-    for (int m = 1; m < 256; m <<= 1) {                   // inclusive scan
+    for (int i = 0; i < kRouteRows / (kPlanT / 64); i++) {
+        const int row = blockIdx.x * kRouteRows + i * (kPlanT / 64) + wave;
+        if (row >= rows) break;
+        route_wave(route + (size_t)row * ld, experts, top, sel[wave], wt[wave]);
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+        if (lane < top) {
+            const int e = sel[wave][lane];
+            pick[row * top + lane] = e;
+            pick_w[row * top + lane] = wt[wave][lane];
+            atomicAdd(&hist[e], 1);
+        }
+        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+    }
+    __syncthreads();
+    for (int e = t; e < experts; e += kPlanT)
+        if (hist[e]) atomicAdd(&counts[e], hist[e]);
+}
+// Place every (row, choice) in its expert's run: a workgroup reserves room for its entries with one atomic per expert.
+// Workgroup 0 also cuts the runs into tiles.
+static __global__ __launch_bounds__(kPlanT) void moe_place_kernel(int rows, int experts, int top, int tile_rows, const int* __restrict__ pick,
+                                                                  int* __restrict__ counts, int* __restrict__ pos_of, int* __restrict__ row_src,
+                                                                  int4* __restrict__ tiles, int* __restrict__ n_tiles) {
+    __shared__ int first[kMaxExperts], tile0[kMaxExperts], hist[kMaxExperts];
+    __shared__ int part[kPlanT], part_t[kPlanT];
+    const int t = threadIdx.x;
+    static_assert(kPlanT >= kMaxExperts, "one thread per expert");
+    const int n = t < experts ? counts[t] : 0, nt = (n + tile_rows - 1) / tile_rows;
+    part[t] = n; part_t[t] = nt;
+    if (t < experts) hist[t] = 0;
+    __syncthreads();
+    for (int m = 1; m < kPlanT; m <<= 1) {                // inclusive scan
         const int a = t >= m ? part[t - m] : 0, b = t >= m ? part_t[t - m] : 0;
         __syncthreads();
         part[t] += a; part_t[t] += b;
         __syncthreads();
     }
-    int o = part[t] - s, ot = part_t[t] - st;
-    for (int i = 0; i < per; i++) {
-        const int e = t * per + i;
-        if (e < experts) { first[e] = o; tile0[e] = ot; o += counts[e]; ot += (counts[e] + tile_rows - 1) / tile_rows; }
-    }
+    const int idx = blockIdx.x * kPlanT + t, e = idx < rows * top ? pick[idx] : -1;
+    const int local = e >= 0 ? atomicAdd(&hist[e], 1) : 0;
+    if (t < experts) tile0[t] = part_t[t] - nt;
     __syncthreads();
-    const int idx = blockIdx.x * 256 + t;
-    if (idx < rows * top) {
-        const int e = pick[idx];
-        const int pos = first[e] + atomicAdd(&counts[experts + e], 1);
+    if (t < experts) first[t] = part[t] - n + (hist[t] ? atomicAdd(&counts[experts + t], hist[t]) : 0);
+    __syncthreads();
+    if (e >= 0) {
+        const int pos = first[e] + local;
         pos_of[idx] = pos;
         row_src[pos] = idx / top;
     }
     if (blockIdx.x == 0) {
-        for (int e = t; e < experts; e += 256) {
-            const int n = counts[e];
-            for (int i = 0; i * tile_rows < n; i++)
-                tiles[tile0[e] + i] = make_int4(e, first[e] + i * tile_rows, first[e] + min(n, (i + 1) * tile_rows), 0);
-        }
-        if (t == 0) n_tiles[0] = part_t[255];
+        if (t < experts)
+            for (int i = 0; i < nt; i++) tiles[tile0[t] + i] = make_int4(t, part[t] - n + i * tile_rows, part[t] - n + min(n, (i + 1) * tile_rows), 0);
+        if (t == 0) n_tiles[0] = part_t[kPlanT - 1];
     }
 }
 
@@ -324,8 +386,8 @@ int moe_plan(const float* route, int ld_route, int rows, int experts, int top, i
     FX_REQUIRE(experts > 0 && experts <= kMaxExperts && top > 0 && top <= kMaxTop && top <= experts, "moe_plan: %d experts, top %d (at most %d, %d)",
                experts, top, kMaxExperts, kMaxTop);
     moe_clear_kernel<<<1, 256, 0, st>>>(p.counts, 2 * experts);
-    moe_route_kernel<<<(rows + 3) / 4, 256, 0, st>>>(route, ld_route, rows, experts, top, p.pick, p.pick_w, p.counts);
-    moe_place_kernel<<<(rows * top + 255) / 256, 256, 0, st>>>(rows, experts, top, tile_rows, p.pick, p.counts, p.pos_of, p.row_src, p.tiles, p.n_tiles);
+    moe_route_kernel<<<(rows + kRouteRows - 1) / kRouteRows, kPlanT, 0, st>>>(route, ld_route, rows, experts, top, p.pick, p.pick_w, p.counts);
+    moe_place_kernel<<<(rows * top + kPlanT - 1) / kPlanT, kPlanT, 0, st>>>(rows, experts, top, tile_rows, p.pick, p.counts, p.pos_of, p.row_src, p.tiles, p.n_tiles);
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
 }

@@ -437,8 +437,8 @@ static int run_small(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T,
         if (layers_out && i > 0) FX_HIP(hipMemcpyAsync(layers_out + (size_t)(i - 1) * T * W, x, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
         if (L.d.mixer == FLEXLLM_MIX_LATENT) {
             ET* rows = static_cast<ET*>(s.rows[i]);
-            FX_TRY(latent_store<ET>(L.ld, m->proj, m->max_et, 1, nf ? m->f32 : nullptr, nf, L.latent_norm, L.cos_t, L.sin_t, rows, s.pos, T, st));
-            FX_TRY(latent_absorbed<ET>(L.ld, m->proj, m->max_et, 1, static_cast<ET*>(L.uk), static_cast<ET*>(L.uv), rows, s.pos, 0, T, m->scratch, m->att, m->max_att, 1, st));
+            FX_TRY(latent_decode<ET>(L.ld, m->proj, m->max_et, nf ? m->f32 : nullptr, nf, L.latent_norm, L.cos_t, L.sin_t, static_cast<ET*>(L.uk),
+                                     static_cast<ET*>(L.uv), rows, s.pos, T, m->scratch, m->att, m->max_att, st));
         } else {
             FX_TRY(gla_steps<ET>(L.gd, m->proj, m->max_et, 1, m->f32, nf, static_cast<ET*>(L.a2), L.a2_bias, L.head_norm, s.state[i], s.pos, 0, T, m->att, m->max_att, 1, st));
         }
@@ -527,7 +527,7 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
         ET *proj = static_cast<ET*>(m->lproj), *att = static_cast<ET*>(m->latt);
         if (L.d.mixer == FLEXLLM_MIX_LATENT) {
             ET *cache = static_cast<ET*>(s.rows[i]), *uk = static_cast<ET*>(L.uk), *uv = static_cast<ET*>(L.uv);
-            FX_TRY(latent_store<ET>(L.ld, proj, ldp, 0, nf ? m->lf32 : nullptr, nf, L.latent_norm, L.cos_t, L.sin_t, cache, s.pos, T, st));
+            FX_TRY(latent_store<ET>(L.ld, proj, ldp, nf ? m->lf32 : nullptr, nf, L.latent_norm, L.cos_t, L.sin_t, cache, s.pos, T, st));
             bool flash = false;
             if constexpr (std::is_same<ET, bf16_t>::value) {
                 flash = latent_flash_ok(L.ld);
@@ -548,7 +548,7 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
             if (!flash)
                 for (int t0 = 0; t0 < T; t0 += kAbsorbTokens) {
                     const int n = T - t0 < kAbsorbTokens ? T - t0 : kAbsorbTokens;
-                    FX_TRY(latent_absorbed<ET>(L.ld, proj + (size_t)t0 * ldp, ldp, 0, uk, uv, cache, s.pos, t0, n, m->scratch, att + (size_t)t0 * lda, lda, 0, st));
+                    FX_TRY(latent_absorbed<ET>(L.ld, proj + (size_t)t0 * ldp, ldp, uk, uv, cache, s.pos, t0, n, m->scratch, att + (size_t)t0 * lda, lda, st));
                 }
         } else if (gla_chunks_ok(L.gd)) {
             FX_TRY(gla_chunks<ET>(L.gd, proj, ldp, m->lf32, nf, static_cast<ET*>(L.a2), L.a2_bias, L.head_norm, s.state[i], s.pos, T, m->lgla, att, lda, st));

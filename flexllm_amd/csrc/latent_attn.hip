@@ -11,8 +11,8 @@
 namespace fx {
 
 // ---- rows of a step into the cache, rotation of the queries -----------------------------------------------------
-template <typename ET, typename QT>
-__global__ __launch_bounds__(256) void latent_store_kernel(LatentDims d, QT* __restrict__ q, int ldq, const float* __restrict__ raw, int ld_raw,
+template <typename ET>
+__global__ __launch_bounds__(256) void latent_store_kernel(LatentDims d, ET* __restrict__ q, int ldq, const float* __restrict__ raw, int ld_raw,
                                                            const float* __restrict__ norm_w, const float* __restrict__ cos_t,
                                                            const float* __restrict__ sin_t, ET* __restrict__ cache, const int* __restrict__ state) {
     __shared__ float red[4];
@@ -33,28 +33,27 @@ __global__ __launch_bounds__(256) void latent_store_kernel(LatentDims d, QT* __r
             row[d.kvp + 2 * i + 1] = (ET)(v * cs[i] + u * sn[i]);
         }
     }
-    QT* qr = q + (size_t)tok * ldq;
+    ET* qr = q + (size_t)tok * ldq;
     const int step = d.dim + d.rot_dim;
     for (int i = t; i < d.heads * rh; i += 256) {
         const int h = i / rh, j = i - h * rh;
-        QT* p = qr + h * step + d.dim + 2 * j;
+        ET* p = qr + h * step + d.dim + 2 * j;
         const float u = (float)p[0], v = (float)p[1];
-        p[0] = (QT)(u * cs[j] - v * sn[j]);
-        p[1] = (QT)(v * cs[j] + u * sn[j]);
+        p[0] = (ET)(u * cs[j] - v * sn[j]);
+        p[1] = (ET)(v * cs[j] + u * sn[j]);
     }
 }
 
 template <typename ET>
-int latent_store(const LatentDims& d, void* q, int ldq, int q_f32, const float* raw, int ld_raw, const float* norm_w, const float* cos_t,
+int latent_store(const LatentDims& d, ET* q, int ldq, const float* raw, int ld_raw, const float* norm_w, const float* cos_t,
                  const float* sin_t, ET* cache, const int* state, int tokens, hipStream_t st) {
     FX_REQUIRE(q && cos_t && sin_t && state && tokens > 0 && (!raw || (cache && norm_w)), "latent_store: null pointer");
-    if (q_f32) latent_store_kernel<ET, float><<<tokens, 256, 0, st>>>(d, static_cast<float*>(q), ldq, raw, ld_raw, norm_w, cos_t, sin_t, cache, state);
-    else latent_store_kernel<ET, ET><<<tokens, 256, 0, st>>>(d, static_cast<ET*>(q), ldq, raw, ld_raw, norm_w, cos_t, sin_t, cache, state);
+    latent_store_kernel<ET><<<tokens, 256, 0, st>>>(d, q, ldq, raw, ld_raw, norm_w, cos_t, sin_t, cache, state);
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
 }
-template int latent_store<bf16_t>(const LatentDims&, void*, int, int, const float*, int, const float*, const float*, const float*, bf16_t*, const int*, int, hipStream_t);
-template int latent_store<float>(const LatentDims&, void*, int, int, const float*, int, const float*, const float*, const float*, float*, const int*, int, hipStream_t);
+template int latent_store<bf16_t>(const LatentDims&, bf16_t*, int, const float*, int, const float*, const float*, const float*, bf16_t*, const int*, int, hipStream_t);
+template int latent_store<float>(const LatentDims&, float*, int, const float*, int, const float*, const float*, const float*, float*, const int*, int, hipStream_t);
 
 // ---- attention in the latent space --------------------------------------------------------------------------------
 constexpr int kAbsCols = 128;                             // latent columns per workgroup of the query kernel
@@ -72,13 +71,13 @@ size_t latent_absorbed_scratch(const LatentDims& d) {
     return (size_t)d.heads * d.ldc + (size_t)d.heads * latent_splits(d).count * (d.kvp + 2);
 }
 
-template <typename ET, typename QT>
-__global__ __launch_bounds__(256) void latent_query_kernel(LatentDims d, const QT* __restrict__ q, int ldq, const ET* __restrict__ w_uk,
+template <typename ET>
+__global__ __launch_bounds__(256) void latent_query_kernel(LatentDims d, const ET* __restrict__ q, int ldq, const ET* __restrict__ w_uk,
                                                            float* __restrict__ ql, int slices) {
     constexpr int CE = Chunk<ET>::N, NC = kAbsCols / CE, NG = 256 / NC;
     __shared__ float part[NG][kAbsCols];
     const int t = threadIdx.x, h = blockIdx.x / slices, c0 = (blockIdx.x % slices) * kAbsCols, tok = blockIdx.y;
-    const QT* qh = q + (size_t)tok * ldq + h * (d.dim + d.rot_dim);
+    const ET* qh = q + (size_t)tok * ldq + h * (d.dim + d.rot_dim);
     float* out = ql + ((size_t)tok * d.heads + h) * d.ldc;
     const int c = t % NC, g = t / NC, col = c0 + c * CE;
     float acc[CE];
@@ -108,6 +107,74 @@ __global__ __launch_bounds__(256) void latent_query_kernel(LatentDims d, const Q
         for (int i = t; i < d.ldc - d.kvp; i += 256) out[d.kvp + i] = i < d.rot_dim ? (float)qh[d.dim + i] : 0.0f;
 }
 
+// The query kernel of a decode step, which also leaves the tokens' own rows in the cache: workgroups 0 .. heads * slices - 1
+// carry the queries over (rotating their rotated part on the way), the last one stores the row.
+template <typename ET>
+__global__ __launch_bounds__(256) void latent_store_query_kernel(LatentDims d, const float* __restrict__ q, int ldq, const float* __restrict__ raw, int ld_raw,
+                                                                 const float* __restrict__ norm_w, const float* __restrict__ cos_t,
+                                                                 const float* __restrict__ sin_t, ET* __restrict__ cache, const int* __restrict__ state,
+                                                                 const ET* __restrict__ w_uk, float* __restrict__ ql, int slices) {
+    constexpr int CE = Chunk<ET>::N, NC = kAbsCols / CE, NG = 256 / NC;
+    __shared__ float part[NG][kAbsCols];
+    __shared__ float red[4];
+    const int t = threadIdx.x, tok = blockIdx.y, rh = d.rot_dim >> 1;
+    const int h = blockIdx.x / slices, slice = blockIdx.x % slices;
+    if (h == d.heads) {
+        const int pos = state[0] + tok;
+        if (!raw || pos >= d.capacity) return;
+        const float* x = raw + (size_t)tok * ld_raw;
+        ET* row = cache + (size_t)pos * d.ldc;
+        float ss = 0.0f;
+        for (int i = t; i < d.kv_rank; i += 256) ss = fma_f(x[i], x[i], ss);
+        const float rs = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)d.kv_rank + d.eps);
+        for (int i = t; i < d.kv_rank; i += 256) row[i] = (ET)(x[i] * rs * norm_w[i]);
+        for (int i = t; i < rh; i += 256) {
+            const float u = x[d.kv_rank + 2 * i], v = x[d.kv_rank + 2 * i + 1], c = cos_t[(size_t)pos * rh + i], s = sin_t[(size_t)pos * rh + i];
+            row[d.kvp + 2 * i] = (ET)(u * c - v * s);
+            row[d.kvp + 2 * i + 1] = (ET)(v * c + u * s);
+        }
+        return;
+    }
+    const float* qh = q + (size_t)tok * ldq + h * (d.dim + d.rot_dim);
+    float* out = ql + ((size_t)tok * d.heads + h) * d.ldc;
+    const int c = t % NC, g = t / NC, c0 = slice * kAbsCols, col = c0 + c * CE;
+    float acc[CE];
+#pragma unroll
+    for (int e = 0; e < CE; e++) acc[e] = 0.0f;
+    if (col < d.kvp) {
+#pragma unroll 8
+        for (int i = g; i < d.dim; i += NG) {
+            const uint4 u = *reinterpret_cast<const uint4*>(w_uk + ((size_t)h * d.dim + i) * d.kvp + col);
+            float wv[CE];
+            Chunk<ET>::unpack(u, wv);
+            const float qv = qh[i];
+#pragma unroll
+            for (int e = 0; e < CE; e++) acc[e] = fma_f(wv[e], qv, acc[e]);
+        }
+    }
+#pragma unroll
+    for (int e = 0; e < CE; e++) part[g][c * CE + e] = acc[e];
+    __syncthreads();
+    if (t < kAbsCols && c0 + t < d.kvp) {
+        float s = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NG; i++) s += part[i][t];
+        out[c0 + t] = s;
+    }
+    if (slice == 0) {
+        const int pos = min(state[0] + tok, d.capacity - 1);
+        for (int i = t; i < d.ldc - d.kvp; i += 256) {
+            float v = 0.0f;
+            if (i < d.rot_dim) {
+                const int j = i >> 1;
+                const float a = qh[d.dim + 2 * j], b = qh[d.dim + 2 * j + 1], cs = cos_t[(size_t)pos * rh + j], sn = sin_t[(size_t)pos * rh + j];
+                v = i & 1 ? b * cs + a * sn : a * cs - b * sn;
+            }
+            out[d.kvp + i] = v;
+        }
+    }
+}
+
 // One split of the visible keys of one (token, head): scores, their maximum and sum, and the weighted sum of latents.
 template <typename ET>
 __global__ __launch_bounds__(256) void latent_split_kernel(LatentDims d, const float* __restrict__ ql, const ET* __restrict__ cache,
@@ -127,26 +194,27 @@ __global__ __launch_bounds__(256) void latent_split_kernel(LatentDims d, const f
     const ET* base = cache + (size_t)first * d.ldc;
     const int nch = d.ldc / CE;
     float mx = -INFINITY;
-    for (int k0 = wave * 4; k0 < n; k0 += 16) {
-        float acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+    constexpr int KW = 8;                                 // keys of a wave in flight
+    for (int k0 = wave * KW; k0 < n; k0 += 4 * KW) {
+        float acc[KW] = {0, 0, 0, 0, 0, 0, 0, 0};
         for (int c = lane; c < nch; c += 64) {
-            uint4 u[4];
+            uint4 u[KW];
 #pragma unroll
-            for (int i = 0; i < 4; i++) u[i] = *reinterpret_cast<const uint4*>(base + (size_t)min(k0 + i, n - 1) * d.ldc + c * CE);
+            for (int i = 0; i < KW; i++) u[i] = *reinterpret_cast<const uint4*>(base + (size_t)min(k0 + i, n - 1) * d.ldc + c * CE);
             float x[CE];
 #pragma unroll
             for (int e = 0; e < CE; e++) x[e] = sq[c * CE + e];
 #pragma unroll
-            for (int i = 0; i < 4; i++) {
+            for (int i = 0; i < KW; i++) {
                 float kv[CE];
                 Chunk<ET>::unpack(u[i], kv);
 #pragma unroll
                 for (int e = 0; e < CE; e++) acc[i] = fma_f(kv[e], x[e], acc[i]);
             }
         }
-        multi_sum_step<4, 1>(acc, lane);
-        if (lane < 4) {
-            const int k = k0 + multi_row<4>(lane);
+        multi_sum_step<KW, 1>(acc, lane);
+        if (lane < KW) {
+            const int k = k0 + multi_row<KW>(lane);
             const float s = acc[0] * d.scale;
             if (k < n) { sc[k] = s; mx = fmaxf(mx, s); }
         }
@@ -192,27 +260,45 @@ __global__ __launch_bounds__(256) void latent_join_kernel(LatentDims d, const fl
                                                           OT* __restrict__ o, int ldo) {
     constexpr int CE = Chunk<ET>::N;
     extern __shared__ __attribute__((aligned(16))) float ctx[];
+    __shared__ float wsp[64];
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6, h = blockIdx.x / slices, v0 = (blockIdx.x % slices) * 32, tok = blockIdx.y;
     const int pos = state[0] + tok0 + tok;
     if (pos >= d.capacity) return;
     const int vis = d.window > 0 ? min(pos + 1, d.window) : pos + 1, ns = (vis + keys - 1) / keys;
     const float* p = part + ((size_t)tok * d.heads + h) * splits * (d.kvp + 2);
     const int ld = d.kvp + 2;
-    float m = -INFINITY, l = 0.0f;
-    for (int s = 0; s < ns; s++) m = fmaxf(m, p[s * ld + d.kvp]);
-    for (int s = 0; s < ns; s++) l += p[s * ld + d.kvp + 1] * exp_f<false>(p[s * ld + d.kvp] - m);
-    for (int i = t; i < d.kvp; i += 256) {
-        float c = 0.0f;
-        for (int s = 0; s < ns; s++) c = fma_f(p[s * ld + i], exp_f<false>(p[s * ld + d.kvp] - m), c);
-        ctx[i] = c / l;
+    const int nch = d.kvp / CE, r0 = v0 + wave * 8;
+    auto rows = [&](int c, uint4 (&u)[8]) {
+#pragma unroll
+        for (int i = 0; i < 8; i++) u[i] = *reinterpret_cast<const uint4*>(w_uv + ((size_t)h * d.vdim + min(r0 + i, d.vdim - 1)) * d.kvp + c * CE);
+    };
+    uint4 first[8];                                       // requested before the splits are joined
+    rows(min(lane, nch - 1), first);
+    {
+        // every wave forms the splits' weights, a lane per split (there are at most kMaxSplits <= 64)
+        const float ms = lane < ns ? p[lane * ld + d.kvp] : -INFINITY, ls = lane < ns ? p[lane * ld + d.kvp + 1] : 0.0f;
+        const float m = wave_max(ms);
+        const float w = lane < ns ? exp_f<false>(ms - m) : 0.0f;
+        const float l = wave_sum(ls * w);
+        if (wave == 0) wsp[lane] = w / l;
     }
     __syncthreads();
-    const int nch = d.kvp / CE, r0 = v0 + wave * 8;
+    for (int i = t; i < d.kvp; i += 256) {
+        float c = 0.0f;
+#pragma unroll 8
+        for (int s = 0; s < ns; s++) c = fma_f(p[s * ld + i], wsp[s], c);
+        ctx[i] = c;
+    }
+    __syncthreads();
     float acc[8] = {0, 0, 0, 0, 0, 0, 0, 0};
     for (int c = lane; c < nch; c += 64) {
         uint4 u[8];
+        if (c == lane) {
 #pragma unroll
-        for (int i = 0; i < 8; i++) u[i] = *reinterpret_cast<const uint4*>(w_uv + ((size_t)h * d.vdim + min(r0 + i, d.vdim - 1)) * d.kvp + c * CE);
+            for (int i = 0; i < 8; i++) u[i] = first[i];
+        } else {
+            rows(c, u);
+        }
         float x[CE];
 #pragma unroll
         for (int e = 0; e < CE; e++) x[e] = ctx[c * CE + e];
@@ -232,15 +318,9 @@ __global__ __launch_bounds__(256) void latent_join_kernel(LatentDims d, const fl
 }
 
 template <typename ET>
-int latent_absorbed(const LatentDims& d, const void* q, int ldq, int q_f32, const ET* w_uk, const ET* w_uv, const ET* cache, const int* state,
-                    int tok0, int tokens, float* scratch, void* o, int ldo, int o_f32, hipStream_t st) {
-    FX_REQUIRE(q && w_uk && w_uv && cache && state && scratch && o && tokens > 0, "latent_absorbed: null pointer");
+static int latent_attend(const LatentDims& d, const float* ql, float* part, const ET* w_uv, const ET* cache, const int* state, int tok0, int tokens,
+                         void* o, int ldo, int o_f32, hipStream_t st) {
     const LatentSplits sp = latent_splits(d);
-    float* ql = scratch;
-    float* part = scratch + (size_t)tokens * d.heads * d.ldc;
-    const int slices = (d.kvp + kAbsCols - 1) / kAbsCols;
-    if (q_f32) latent_query_kernel<ET, float><<<dim3(d.heads * slices, tokens), 256, 0, st>>>(d, static_cast<const float*>(q), ldq, w_uk, ql, slices);
-    else latent_query_kernel<ET, ET><<<dim3(d.heads * slices, tokens), 256, 0, st>>>(d, static_cast<const ET*>(q), ldq, w_uk, ql, slices);
     const size_t lds = (size_t)(d.ldc + sp.keys + 256 * Chunk<ET>::N) * sizeof(float);
     FX_REQUIRE(lds <= 60 * 1024 && d.kvp * sizeof(float) <= 60 * 1024, "latent_absorbed: latent of %d (padded) with %d keys per split exceeds LDS", d.kvp, sp.keys);
     latent_split_kernel<ET><<<dim3(sp.count, d.heads, tokens), 256, lds, st>>>(d, ql, cache, state, tok0, sp.keys, sp.count, part);
@@ -250,8 +330,28 @@ int latent_absorbed(const LatentDims& d, const void* q, int ldq, int q_f32, cons
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
 }
-template int latent_absorbed<bf16_t>(const LatentDims&, const void*, int, int, const bf16_t*, const bf16_t*, const bf16_t*, const int*, int, int, float*, void*, int, int, hipStream_t);
-template int latent_absorbed<float>(const LatentDims&, const void*, int, int, const float*, const float*, const float*, const int*, int, int, float*, void*, int, int, hipStream_t);
+
+template <typename ET>
+int latent_absorbed(const LatentDims& d, const ET* q, int ldq, const ET* w_uk, const ET* w_uv, const ET* cache, const int* state,
+                    int tok0, int tokens, float* scratch, ET* o, int ldo, hipStream_t st) {
+    FX_REQUIRE(q && w_uk && w_uv && cache && state && scratch && o && tokens > 0, "latent_absorbed: null pointer");
+    const int slices = (d.kvp + kAbsCols - 1) / kAbsCols;
+    latent_query_kernel<ET><<<dim3(d.heads * slices, tokens), 256, 0, st>>>(d, q, ldq, w_uk, scratch, slices);
+    return latent_attend<ET>(d, scratch, scratch + (size_t)tokens * d.heads * d.ldc, w_uv, cache, state, tok0, tokens, o, ldo, 0, st);
+}
+template int latent_absorbed<bf16_t>(const LatentDims&, const bf16_t*, int, const bf16_t*, const bf16_t*, const bf16_t*, const int*, int, int, float*, bf16_t*, int, hipStream_t);
+template int latent_absorbed<float>(const LatentDims&, const float*, int, const float*, const float*, const float*, const int*, int, int, float*, float*, int, hipStream_t);
+
+template <typename ET>
+int latent_decode(const LatentDims& d, const float* q, int ldq, const float* raw, int ld_raw, const float* norm_w, const float* cos_t, const float* sin_t,
+                  const ET* w_uk, const ET* w_uv, ET* cache, const int* state, int tokens, float* scratch, float* o, int ldo, hipStream_t st) {
+    FX_REQUIRE(q && cos_t && sin_t && w_uk && w_uv && cache && state && scratch && o && tokens > 0 && (!raw || norm_w), "latent_decode: null pointer");
+    const int slices = (d.kvp + kAbsCols - 1) / kAbsCols;
+    latent_store_query_kernel<ET><<<dim3(d.heads * slices + 1, tokens), 256, 0, st>>>(d, q, ldq, raw, ld_raw, norm_w, cos_t, sin_t, cache, state, w_uk, scratch, slices);
+    return latent_attend<ET>(d, scratch, scratch + (size_t)tokens * d.heads * d.ldc, w_uv, cache, state, 0, tokens, o, ldo, 1, st);
+}
+template int latent_decode<bf16_t>(const LatentDims&, const float*, int, const float*, int, const float*, const float*, const float*, const bf16_t*, const bf16_t*, bf16_t*, const int*, int, float*, float*, int, hipStream_t);
+template int latent_decode<float>(const LatentDims&, const float*, int, const float*, int, const float*, const float*, const float*, const float*, const float*, float*, const int*, int, float*, float*, int, hipStream_t);
 
 // ---- attention of many tokens --------------------------------------------------------------------------------------
 // Workgroup: 4 waves x 32 queries of one head over key tiles of 64.  The score tile is formed transposed (keys x
