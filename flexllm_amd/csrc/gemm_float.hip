@@ -234,6 +234,36 @@ static int launch_bf16(const GemmArgs& g, hipStream_t st) {
     return FLEXLLM_OK;
 }
 
+// A few float32 output columns (router rows, low-rank gate inputs): 16 rows x 16 columns per workgroup on
+// v_mfma_f32_16x16x32_bf16, the four waves sharing k; operands straight from memory, eight k-steps in flight.
+__global__ __launch_bounds__(256) void gemm_bf16_narrow_kernel(GemmArgs g, int n0) {
+    __shared__ float part[4][16 * 17];
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, row0 = blockIdx.x * 16, col0 = n0 + blockIdx.y * 16;
+    const int r = min(row0 + (lane & 15), g.m - 1), c = min(col0 + (lane & 15), g.n - 1), kq = (lane >> 4) * 8;
+    const bf16_t* a = static_cast<const bf16_t*>(g.a) + (size_t)r * g.lda + kq;
+    const bf16_t* w = static_cast<const bf16_t*>(g.w) + (size_t)c * g.ldw + kq;
+    f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+    constexpr int B = 8;
+    for (int k0 = wave * 32 * B; k0 < g.k; k0 += 4 * 32 * B) {
+        bf16x8 fa[B], fb[B];
+#pragma unroll
+        for (int i = 0; i < B; i++) {
+            const int k = min(k0 + i * 32, g.k - 32);     // k is a multiple of 64; steps beyond it are left out below
+            fa[i] = *reinterpret_cast<const bf16x8*>(a + k);
+            fb[i] = *reinterpret_cast<const bf16x8*>(w + k);
+        }
+#pragma unroll
+        for (int i = 0; i < B; i++)
+            if (k0 + i * 32 < g.k) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[i], fb[i], acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) part[wave][((lane >> 4) * 4 + i) * 17 + (lane & 15)] = acc[i];
+    __syncthreads();
+    const int rr = t >> 4, cc = t & 15;
+    const float v = (part[0][rr * 17 + cc] + part[1][rr * 17 + cc]) + (part[2][rr * 17 + cc] + part[3][rr * 17 + cc]);
+    if (row0 + rr < g.m && col0 + cc < g.n) g.y32[(size_t)(row0 + rr) * g.ldy32 + (col0 + cc - g.n_split)] = v;
+}
+
 int gemm_group_tile_rows(int rows_per_group) { return rows_per_group >= 96 ? 128 : 64; }
 
 static int gemm_check(GemmArgs& g, size_t a_rows, int es) {
@@ -253,6 +283,13 @@ int gemm_float<bf16_t>(const GemmArgs& args, hipStream_t st) {
     int rc = gemm_check(g, g.m, 2);
     if (rc) return rc;
     FX_REQUIRE(!g.tiles, "gemm_float: a tile table goes to gemm_grouped");
+    // a few float32 columns behind whole tiles would cost a tile column of their own: they get the narrow kernel
+    const int extra = g.n - g.n_split;
+    if (g.n_split > 0 && extra > 0 && extra <= 256 && (g.n + 127) / 128 > (g.n_split + 127) / 128) {
+        gemm_bf16_narrow_kernel<<<dim3((g.m + 15) / 16, (extra + 15) / 16), 256, 0, st>>>(g, g.n_split);
+        FX_LAUNCH_CHECK();
+        g.n = g.n_split;
+    }
     auto tiles = [&](int bm, int bn) { return ((g.m + bm - 1) / bm) * ((g.n + bn - 1) / bn); };
     const int t256 = tiles(256, 256);
     if (t256 >= 256 && (t256 % 256 == 0 || t256 >= 1024)) return launch_bf16<256, 256, 2, 2, 8>(g, st);

@@ -26,7 +26,7 @@ __device__ __forceinline__ void route_wave(const float* __restrict__ z, int expe
     float den = 0.0f;
 #pragma unroll
     for (int i = 0; i < kMaxExperts / 64; i++) {
-        if (i * 64 >= experts) break;
+        if (i * 64 >= experts) continue;
         v[i] = i * 64 + lane < experts ? exp_f(v[i] - mx) : -1.0f;
         den += fmaxf(v[i], 0.0f);
     }
@@ -35,15 +35,13 @@ __device__ __forceinline__ void route_wave(const float* __restrict__ z, int expe
     for (int k = 0; k < top; k++) {
         float best = -2.0f;
 #pragma unroll
-        for (int i = 0; i < kMaxExperts / 64; i++) {
-            if (i * 64 >= experts) break;
-            best = fmaxf(best, v[i]);
-        }
+        for (int i = 0; i < kMaxExperts / 64; i++)
+            if (i * 64 < experts) best = fmaxf(best, v[i]);
         best = wave_max(best);
         int bi = -1;                                      // lowest index that holds the maximum
 #pragma unroll
         for (int i = 0; i < kMaxExperts / 64; i++) {
-            if (i * 64 >= experts) break;
+            if (i * 64 >= experts) continue;
             const unsigned long long hit = __ballot(v[i] == best);
             if (bi < 0 && hit) {
                 const int l = __builtin_ctzll(hit);
@@ -59,9 +57,9 @@ __device__ __forceinline__ void route_wave(const float* __restrict__ z, int expe
         for (int k = 0; k < top; k++) wt[k] = wt[k] / (sum + 1e-20f);
 }
 
-// VQ: the norm prologue keeps its vectors in registers, VQ float4 per thread (k a multiple of 4, at most 1024 VQ); 0: any k,
-// through LDS.  Only used with PRO = 1.
-template <typename ET, int R, int S, int PRO, int VQ>
+// VEC: the prologue keeps its vectors in registers as float4 (k a multiple of 4, at most what the S pieces per thread cover);
+// else any k, through LDS.
+template <typename ET, int R, int S, int PRO, bool VEC>
 __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     constexpr int CE = Chunk<ET>::N;
     extern __shared__ __attribute__((aligned(16))) float xs[];     // [kpad] the vector
@@ -74,21 +72,23 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     const ET* w = static_cast<const ET*>(g.w);
     const float* x = g.x + (size_t)tok * g.ldx;
     // ---- requests for the vector go out first: loads return in order, and the weights behind them are a long stream
-    constexpr int Q = VQ > 0 ? VQ : 1;
+    constexpr int Q = VEC ? S * CE / 4 : 1;               // float4 per thread
     f32x4 xv[Q], yv[Q], gb[Q], gv[Q];
     const int k4 = g.k >> 2;
     const bool have_y = PRO == 1 && g.y != nullptr;
-    if constexpr (PRO == 1 && VQ > 0) {
+    if constexpr (VEC) {
         const f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
         const float* y = g.y + (size_t)tok * g.ldy;
 #pragma unroll
         for (int i = 0; i < Q; i++) {
             const int c = t + 256 * i;
             const bool in = c < k4;
-            yv[i] = in && have_y ? *reinterpret_cast<const f32x4*>(y + 4 * c) : zero;
+            if constexpr (PRO == 1) yv[i] = in && have_y ? *reinterpret_cast<const f32x4*>(y + 4 * c) : zero;
             xv[i] = in ? *reinterpret_cast<const f32x4*>(x + 4 * c) : zero;
-            gb[i] = in && have_y ? *reinterpret_cast<const f32x4*>(g.gb + 4 * c) : zero;
-            gv[i] = in ? *reinterpret_cast<const f32x4*>(g.g + 4 * c) : zero;
+            if constexpr (PRO == 1) {
+                gb[i] = in && have_y ? *reinterpret_cast<const f32x4*>(g.gb + 4 * c) : zero;
+                gv[i] = in ? *reinterpret_cast<const f32x4*>(g.g + 4 * c) : zero;
+            }
         }
         __builtin_amdgcn_sched_barrier(0);
     }
@@ -117,7 +117,7 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     if (g0 + G < ng) load(1, g0 + G);
     __builtin_amdgcn_sched_barrier(0);
     // ---- the vector
-    if constexpr (PRO == 1 && VQ > 0) {
+    if constexpr (PRO == 1 && VEC) {
         float rs = 0.0f;
         if (have_y) {
             float ss = 0.0f;
@@ -170,6 +170,10 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
             xs[i] = v;
             if (blockIdx.x == 0 && g.h_out && i < g.k) g.h_out[(size_t)tok * g.ldh + i] = v;
         }
+    } else if constexpr (VEC) {
+#pragma unroll
+        for (int i = 0; i < Q; i++)
+            if (4 * (t + 256 * i) < g.kpad) *reinterpret_cast<f32x4*>(xs + 4 * (t + 256 * i)) = xv[i];
     } else {
         for (int i = t; i < g.kpad; i += 256) xs[i] = i < g.k ? x[i] : 0.0f;
     }
@@ -235,12 +239,16 @@ static int launch_gemv_rs(const GemvArgs& g, int pro, int rows_y, hipStream_t st
     const int ng = (g.n + R - 1) / R;
     const dim3 grid(ng < wgs ? ng : wgs, rows_y);
     const size_t lds = (size_t)g.kpad * sizeof(float);
-    const bool vec = g.k % 4 == 0 && g.ldx % 4 == 0 && g.ldy % 4 == 0 && g.ldh % 4 == 0;
-    if (pro == 0) gemv_float_kernel<ET, R, S, 0, 0><<<grid, 256, lds, st>>>(g);
-    else if (pro == 2) gemv_float_kernel<ET, R, S, 2, 0><<<grid, 256, lds, st>>>(g);
-    else if (vec && g.kpad <= 2048) gemv_float_kernel<ET, R, S, 1, 2><<<grid, 256, lds, st>>>(g);
-    else if (vec && g.kpad <= 4096) gemv_float_kernel<ET, R, S, 1, 4><<<grid, 256, lds, st>>>(g);
-    else gemv_float_kernel<ET, R, S, 1, 0><<<grid, 256, lds, st>>>(g);
+    const bool vec = g.k % 4 == 0 && g.ldx % 4 == 0 && g.ldy % 4 == 0 && g.ldh % 4 == 0 && g.kpad <= 256 * Chunk<ET>::N * S;
+#define FX_GEMV(PRO)                                                                               \
+    do {                                                                                           \
+        if (vec) gemv_float_kernel<ET, R, S, PRO, true><<<grid, 256, lds, st>>>(g);                \
+        else gemv_float_kernel<ET, R, S, PRO, false><<<grid, 256, lds, st>>>(g);                   \
+    } while (0)
+    if (pro == 0) FX_GEMV(0);
+    else if (pro == 1) FX_GEMV(1);
+    else FX_GEMV(2);
+#undef FX_GEMV
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
 }

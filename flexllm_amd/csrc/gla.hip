@@ -211,33 +211,45 @@ constexpr float kGlaMild = -40.0f;                        // smallest running su
 template <typename ET, int RMAX>
 __global__ __launch_bounds__(256) void gla_cum_kernel(GlaDims d, const float* __restrict__ a1, int ld_a1, const ET* __restrict__ w_a2,
                                                       const float* __restrict__ b_a2, int tokens, int C, float* __restrict__ cum) {
-    extern __shared__ __attribute__((aligned(16))) float s1[];      // [C][rank]
+    constexpr bool kRegs = RMAX > 0;
+    const int rp = kRegs ? RMAX : d.a_rank;               // row length in LDS, zero beyond the rank
+    extern __shared__ __attribute__((aligned(16))) float s1[];
     const int t = threadIdx.x, tok0 = blockIdx.x * C, n = min(C, tokens - tok0), HD = d.heads * d.dim, ch = blockIdx.y * 256 + t;
-    for (int i = t; i < n * d.a_rank; i += 256) s1[i] = a1[(size_t)(tok0 + i / d.a_rank) * ld_a1 + i % d.a_rank];
+    for (int i = t; i < n * rp; i += 256) {
+        const int r = i / rp, c = i - r * rp;
+        s1[i] = c < d.a_rank ? a1[(size_t)(tok0 + r) * ld_a1 + c] : 0.0f;
+    }
+    const ET* w = w_a2 + (size_t)min(ch, HD - 1) * pad_k(d.a_rank);
+    const float b = b_a2[min(ch, HD - 1)], inv = 1.0f / d.tau;
+    float wr[kRegs ? RMAX : 1];
+    if constexpr (kRegs) {                                // the weights' rows are padded with zeros to 64 columns
+        constexpr int CE = Chunk<ET>::N;
+#pragma unroll
+        for (int r = 0; r < RMAX; r += CE) {
+            float v[CE];
+            Chunk<ET>::unpack(*reinterpret_cast<const uint4*>(w + r), v);
+#pragma unroll
+            for (int e = 0; e < CE; e++) wr[r + e] = v[e];
+        }
+    }
     __syncthreads();
     if (ch >= HD) return;
-    const ET* w = w_a2 + (size_t)ch * pad_k(d.a_rank);
-    const float b = b_a2[ch], inv = 1.0f / d.tau;
     float s = 0.0f;
-    if constexpr (RMAX > 0) {
-        float wr[RMAX];
+#pragma unroll 4
+    for (int i = 0; i < n; i++) {
+        float z = b;
+        if constexpr (kRegs) {
 #pragma unroll
-        for (int r = 0; r < RMAX; r++) wr[r] = r < d.a_rank ? (float)w[r] : 0.0f;
-        for (int i = 0; i < n; i++) {
-            float z = b;
+            for (int r = 0; r < RMAX; r += 4) {
+                const f32x4 x = *reinterpret_cast<const f32x4*>(s1 + i * RMAX + r);
 #pragma unroll
-            for (int r = 0; r < RMAX; r++)
-                if (r < d.a_rank) z = fma_f(wr[r], s1[i * d.a_rank + r], z);
-            s += log_sigmoid_f(z) * inv;
-            cum[(size_t)(tok0 + i) * HD + ch] = s;
-        }
-    } else {
-        for (int i = 0; i < n; i++) {
-            float z = b;
+                for (int e = 0; e < 4; e++) z = fma_f(wr[r + e], x[e], z);
+            }
+        } else {
             for (int r = 0; r < d.a_rank; r++) z = fma_f((float)w[r], s1[i * d.a_rank + r], z);
-            s += log_sigmoid_f(z) * inv;
-            cum[(size_t)(tok0 + i) * HD + ch] = s;
         }
+        s += log_sigmoid_f(z) * inv;
+        cum[(size_t)(tok0 + i) * HD + ch] = s;
     }
 }
 
@@ -676,7 +688,7 @@ static int gla_chunks_c(const GlaDims& d, const ET* p, int ldp, const float* a1,
     int rc;
     {
         const dim3 grid(nc, (HD + 255) / 256);
-        const size_t lds = sizeof(float) * C * d.a_rank;
+        const size_t lds = sizeof(float) * C * (d.a_rank <= 16 ? 16 : d.a_rank <= 32 ? 32 : d.a_rank);
         if (d.a_rank <= 16) gla_cum_kernel<ET, 16><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, C, cum);
         else if (d.a_rank <= 32) gla_cum_kernel<ET, 32><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, C, cum);
         else gla_cum_kernel<ET, 0><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, C, cum);

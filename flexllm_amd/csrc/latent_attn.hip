@@ -253,6 +253,101 @@ __global__ __launch_bounds__(256) void latent_split_kernel(LatentDims d, const f
     }
 }
 
+// The same with the split's rows staged in LDS, tile by tile (TK rows), so that the cache is read in one burst per tile and
+// both passes over a tile run from LDS; sums of earlier tiles are rescaled as the maximum grows.  A thread owns the latent
+// columns of piece t % ncl for every G-th row.
+constexpr int kSplitPieces = 20;                          // 16-byte pieces in flight per thread
+template <typename ET>
+__global__ __launch_bounds__(256) void latent_split_tile_kernel(LatentDims d, const float* __restrict__ ql, const ET* __restrict__ cache,
+                                                                const int* __restrict__ state, int tok0, int keys, int splits, int tk, float* __restrict__ part) {
+    constexpr int CE = Chunk<ET>::N, KW = 4;
+    extern __shared__ __attribute__((aligned(16))) int8_t sm8[];   // rows [tk][ldc] of ET, q [ldc], weights [tk], sums [256 * CE]
+    __shared__ float red[4];
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, h = blockIdx.y, tok = blockIdx.z;
+    ET* rows = reinterpret_cast<ET*>(sm8);
+    float* sq = reinterpret_cast<float*>(sm8 + (size_t)tk * d.ldc * sizeof(ET));
+    float *sc = sq + d.ldc, *sum = sc + tk;
+    const float* qv = ql + ((size_t)tok * d.heads + h) * d.ldc;
+    const int pos = state[0] + tok0 + tok;
+    for (int i = t; i < d.ldc; i += 256) sq[i] = qv[i];
+    const int lo = d.window > 0 && pos - d.window + 1 > 0 ? pos - d.window + 1 : 0;
+    const int first = lo + blockIdx.x * keys, n = min(keys, pos + 1 - first);
+    if (n <= 0 || pos >= d.capacity) return;
+    const int nch = d.ldc / CE, ncl = d.kvp / CE, groups = 256 / ncl, c = t % ncl, g = t / ncl;
+    float m = -INFINITY, l = 0.0f, acc[CE];
+#pragma unroll
+    for (int e = 0; e < CE; e++) acc[e] = 0.0f;
+    for (int k0 = 0; k0 < n; k0 += tk) {
+        const int nk = min(tk, n - k0), total = nk * nch;
+        const i32x4* src = reinterpret_cast<const i32x4*>(cache + (size_t)(first + k0) * d.ldc);    // the rows are one run of memory
+        i32x4* dst = reinterpret_cast<i32x4*>(rows);
+        __syncthreads();                                  // the previous tile has been read; q is in
+        for (int b = 0; b < total; b += 256 * kSplitPieces) {
+            i32x4 u[kSplitPieces];
+#pragma unroll
+            for (int i = 0; i < kSplitPieces; i++) u[i] = src[min(b + 256 * i + t, total - 1)];
+#pragma unroll
+            for (int i = 0; i < kSplitPieces; i++)
+                if (b + 256 * i + t < total) dst[b + 256 * i + t] = u[i];
+        }
+        __syncthreads();
+        float mx = -INFINITY;
+        for (int k = wave * KW; k < nk; k += 4 * KW) {
+            float a[KW] = {0, 0, 0, 0};
+            for (int cc = lane; cc < nch; cc += 64) {
+                float x[CE];
+#pragma unroll
+                for (int q4 = 0; q4 < CE / 4; q4++) {
+                    const f32x4 v = *reinterpret_cast<const f32x4*>(sq + cc * CE + q4 * 4);
+#pragma unroll
+                    for (int e = 0; e < 4; e++) x[q4 * 4 + e] = v[e];
+                }
+#pragma unroll
+                for (int i = 0; i < KW; i++) {
+                    float kv[CE];
+                    Chunk<ET>::unpack(*reinterpret_cast<const uint4*>(rows + (size_t)min(k + i, nk - 1) * d.ldc + cc * CE), kv);
+#pragma unroll
+                    for (int e = 0; e < CE; e++) a[i] = fma_f(kv[e], x[e], a[i]);
+                }
+            }
+            multi_sum_step<KW, 1>(a, lane);
+            if (lane < KW) {
+                const int key = k + multi_row<KW>(lane);
+                const float s = a[0] * d.scale;
+                if (key < nk) { sc[key] = s; mx = fmaxf(mx, s); }
+            }
+        }
+        mx = fmaxf(m, block_max<4>(mx, red));
+        const float al = k0 == 0 ? 0.0f : exp_f<false>(m - mx);
+        m = mx;
+        float ls = 0.0f;
+        if (t < nk) { const float p = exp_f<false>(sc[t] - mx); sc[t] = p; ls = p; }
+        l = l * al + block_sum<4>(ls, red);
+#pragma unroll
+        for (int e = 0; e < CE; e++) acc[e] *= al;
+        if (g < groups)
+#pragma unroll 4
+            for (int k = g; k < nk; k += groups) {
+                float kv[CE];
+                Chunk<ET>::unpack(*reinterpret_cast<const uint4*>(rows + (size_t)k * d.ldc + c * CE), kv);
+                const float p = sc[k];
+#pragma unroll
+                for (int e = 0; e < CE; e++) acc[e] = fma_f(p, kv[e], acc[e]);
+            }
+    }
+    float* out = part + (((size_t)tok * d.heads + h) * splits + blockIdx.x) * (d.kvp + 2);
+    if (t == 0) { out[d.kvp] = m; out[d.kvp + 1] = l; }
+    if (g < groups)
+#pragma unroll
+        for (int e = 0; e < CE; e++) sum[(g * ncl + c) * CE + e] = acc[e];
+    __syncthreads();
+    for (int i = t; i < d.kvp; i += 256) {
+        float s = 0.0f;
+        for (int j = 0; j < groups; j++) s += sum[j * d.kvp + i];
+        out[i] = s;
+    }
+}
+
 // Join the splits of one (token, head) and carry the context back: 32 value rows per workgroup.
 template <typename ET, typename OT>
 __global__ __launch_bounds__(256) void latent_join_kernel(LatentDims d, const float* __restrict__ part, const ET* __restrict__ w_uv,
@@ -321,9 +416,17 @@ template <typename ET>
 static int latent_attend(const LatentDims& d, const float* ql, float* part, const ET* w_uv, const ET* cache, const int* state, int tok0, int tokens,
                          void* o, int ldo, int o_f32, hipStream_t st) {
     const LatentSplits sp = latent_splits(d);
-    const size_t lds = (size_t)(d.ldc + sp.keys + 256 * Chunk<ET>::N) * sizeof(float);
+    size_t lds = (size_t)(d.ldc + sp.keys + 256 * Chunk<ET>::N) * sizeof(float);
     FX_REQUIRE(lds <= 60 * 1024 && d.kvp * sizeof(float) <= 60 * 1024, "latent_absorbed: latent of %d (padded) with %d keys per split exceeds LDS", d.kvp, sp.keys);
-    latent_split_kernel<ET><<<dim3(sp.count, d.heads, tokens), 256, lds, st>>>(d, ql, cache, state, tok0, sp.keys, sp.count, part);
+    int tk = 64;                                          // rows per tile: at most 76 KiB, two workgroups per CU
+    while (tk > 8 && (size_t)tk * d.ldc * sizeof(ET) > 76 * 1024) tk /= 2;
+    if (d.kvp <= 256 * Chunk<ET>::N && (size_t)tk * d.ldc * sizeof(ET) <= 76 * 1024) {
+        lds = (size_t)tk * d.ldc * sizeof(ET) + (size_t)(d.ldc + tk + 256 * Chunk<ET>::N) * sizeof(float);
+        FX_HIP(hipFuncSetAttribute(reinterpret_cast<const void*>(latent_split_tile_kernel<ET>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+        latent_split_tile_kernel<ET><<<dim3(sp.count, d.heads, tokens), 256, lds, st>>>(d, ql, cache, state, tok0, sp.keys, sp.count, tk, part);
+    } else {
+        latent_split_kernel<ET><<<dim3(sp.count, d.heads, tokens), 256, lds, st>>>(d, ql, cache, state, tok0, sp.keys, sp.count, part);
+    }
     const int vs = (d.vdim + 31) / 32;
     if (o_f32) latent_join_kernel<ET, float><<<dim3(d.heads * vs, tokens), 256, d.kvp * sizeof(float), st>>>(d, part, w_uv, state, tok0, sp.keys, sp.count, vs, static_cast<float*>(o), ldo);
     else latent_join_kernel<ET, ET><<<dim3(d.heads * vs, tokens), 256, d.kvp * sizeof(float), st>>>(d, part, w_uv, state, tok0, sp.keys, sp.count, vs, static_cast<ET*>(o), ldo);
@@ -354,19 +457,22 @@ template int latent_decode<bf16_t>(const LatentDims&, const float*, int, const f
 template int latent_decode<float>(const LatentDims&, const float*, int, const float*, int, const float*, const float*, const float*, const float*, const float*, float*, const int*, int, float*, float*, int, hipStream_t);
 
 // ---- attention of many tokens --------------------------------------------------------------------------------------
-// Workgroup: 4 waves x 32 queries of one head over key tiles of 64.  The score tile is formed transposed (keys x
+// Workgroup: NW waves x 32 queries of one head over key tiles of 64.  The score tile is formed transposed (keys x
 // queries), so that a lane holds one query's scores, and its registers are already the operand of the second product:
 // the slots of that product's k dimension are assigned to the keys in accumulator order (slot j of half-wave h = key
 // 8 * (j / 4) + 4 * h + j % 4 of each 16), which the reads of the transposed values follow.
 // LDS: keys in planes of 8 dims [plane][64 keys][16 B], values in planes of 4 keys [plane][value row][8 B].
-constexpr int kFlashQ = 128, kFlashK = 64;
+// Planes beyond a head's own dims meet zeros on the query side, value rows beyond vdim are not stored: both may hold any
+// finite value, so no load is conditional.
+constexpr int kFlashK = 64;
 
-template <int DK, int DV>
-__global__ __launch_bounds__(256, DV > 128 ? 1 : 2) void latent_flash_kernel(LatentDims d, const bf16_t* __restrict__ q, int ldq, const bf16_t* __restrict__ k, int ldk,
+template <int DK, int DV, int NW>
+__global__ __launch_bounds__(NW * 64, (DV > 128 || NW < 4) ? 1 : 2) void latent_flash_kernel(LatentDims d, const bf16_t* __restrict__ q, int ldq, const bf16_t* __restrict__ k, int ldk,
                                                            const bf16_t* __restrict__ vt, int ldv, const bf16_t* __restrict__ cache, int kv0, int pos0,
                                                            int tokens, int rows, bf16_t* __restrict__ o, int ldo) {
     constexpr int NP = DK / 8, KP = kFlashK * 16 + 32, VP = DV * 8 + 16, NVT = DV / 32;
-    constexpr int KCH = NP * kFlashK / 256, VCH = DV * 8 / 256;          // 16-byte pieces per thread and tile
+    constexpr int T = NW * 64, kFlashQ = NW * 32;
+    constexpr int KCH = NP * kFlashK / T, VCH = DV * 8 / T;              // 16-byte pieces per thread and tile
     __shared__ __attribute__((aligned(16))) int8_t lk[NP * KP];
     __shared__ __attribute__((aligned(16))) int8_t lv[16 * VP];
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6, half = lane >> 5, ln = lane & 31;
@@ -399,34 +505,42 @@ __global__ __launch_bounds__(256, DV > 128 ? 1 : 2) void latent_flash_kernel(Lat
     const int qp = pos0 + wq0 + ln;                       // this lane's position
     const int qmin = pos0 + wq0, qmax = pos0 + wq0 + 31;
 
-    uint4 rk[KCH], rv[VCH];
+    i32x4 rk[KCH], rv[VCH];
+    const bf16_t* kbase[KCH];                             // row 0 of the piece's source, its row and row length
+    int krow[KCH], kld[KCH], voff[VCH];
+#pragma unroll
+    for (int i = 0; i < KCH; i++) {
+        const int c = t + T * i, pl = c % NP;
+        const bool rot = pl >= dim8 && (pl - dim8) * 8 < d.rot_dim;
+        kbase[i] = rot ? cache + (size_t)kv0 * d.ldc + d.kvp + (pl - dim8) * 8 : k + h * d.dim + (pl * 8 < d.dim ? pl * 8 : 0);
+        krow[i] = c / NP;
+        kld[i] = rot ? d.ldc : ldk;
+    }
+#pragma unroll
+    for (int i = 0; i < VCH; i++) {
+        const int c = t + T * i;
+        voff[i] = min(c >> 3, d.vdim - 1) * ldv + (c & 7) * 8;
+    }
+    const bf16_t* vh = vt + (size_t)h * d.vdim * ldv;
     auto load = [&](int kb) {
 #pragma unroll
-        for (int i = 0; i < KCH; i++) {
-            const int c = t + 256 * i, pl = c % NP, key = min(kb + c / NP, rows - 1);
-            rk[i] = zero;
-            if (pl < dim8) { if (pl * 8 < d.dim) rk[i] = *reinterpret_cast<const uint4*>(k + (size_t)key * ldk + h * d.dim + pl * 8); }
-            else if ((pl - dim8) * 8 < d.rot_dim) rk[i] = *reinterpret_cast<const uint4*>(cache + (size_t)(kv0 + key) * d.ldc + d.kvp + (pl - dim8) * 8);
-        }
+        for (int i = 0; i < KCH; i++) rk[i] = *reinterpret_cast<const i32x4*>(kbase[i] + (size_t)(unsigned)(min(kb + krow[i], rows - 1) * kld[i]));
 #pragma unroll
-        for (int i = 0; i < VCH; i++) {
-            const int c = t + 256 * i, v = c >> 3;
-            rv[i] = v < d.vdim ? *reinterpret_cast<const uint4*>(vt + (size_t)(h * d.vdim + v) * ldv + kb + (c & 7) * 8) : zero;
-        }
+        for (int i = 0; i < VCH; i++) rv[i] = *reinterpret_cast<const i32x4*>(vh + kb + voff[i]);
     };
     load(kb0);
     for (int kb = kb0; kb <= kb1; kb += kFlashK) {
         __syncthreads();
 #pragma unroll
         for (int i = 0; i < KCH; i++) {
-            const int c = t + 256 * i;
-            *reinterpret_cast<uint4*>(lk + (c % NP) * KP + (c / NP) * 16) = rk[i];
+            const int c = t + T * i;
+            *reinterpret_cast<i32x4*>(lk + (c % NP) * KP + krow[i] * 16) = rk[i];
         }
 #pragma unroll
         for (int i = 0; i < VCH; i++) {
-            const int c = t + 256 * i;
-            *reinterpret_cast<uint2*>(lv + ((c & 7) * 2) * VP + (c >> 3) * 8) = make_uint2(rv[i].x, rv[i].y);
-            *reinterpret_cast<uint2*>(lv + ((c & 7) * 2 + 1) * VP + (c >> 3) * 8) = make_uint2(rv[i].z, rv[i].w);
+            const int c = t + T * i;
+            *reinterpret_cast<int2*>(lv + ((c & 7) * 2) * VP + (c >> 3) * 8) = make_int2(rv[i][0], rv[i][1]);
+            *reinterpret_cast<int2*>(lv + ((c & 7) * 2 + 1) * VP + (c >> 3) * 8) = make_int2(rv[i][2], rv[i][3]);
         }
         __syncthreads();
         if (kb + kFlashK <= kb1) load(kb + kFlashK);
@@ -444,21 +558,26 @@ __global__ __launch_bounds__(256, DV > 128 ? 1 : 2) void latent_flash_kernel(Lat
                 const bf16x8 fk = *reinterpret_cast<const bf16x8*>(lk + (st * 2 + half) * KP + (j * 32 + ln) * 16);
                 s[j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fk, fq[st], s[j], 0, 0, 0);
             }
-        const bool edge = kp + kFlashK - 1 > qmin || (d.window > 0 && kp < qmax - d.window + 1);
         float mx = m;
+        if (kp + kFlashK - 1 > qmin || (d.window > 0 && kp < qmax - d.window + 1)) {     // the tile holds unseen keys
+            const int far = d.window > 0 ? d.window : 0x7fffffff;
 #pragma unroll
-        for (int j = 0; j < 2; j++)
+            for (int j = 0; j < 2; j++)
 #pragma unroll
-            for (int r = 0; r < 16; r++) {
-                float v = s[j][r] * sc2;
-                if (edge) {
-                    const int key = kp + j * 32 + (r >> 2) * 8 + half * 4 + (r & 3);
-                    const bool seen = key <= qp && (d.window <= 0 || qp - key < d.window);
-                    v = seen ? v : -INFINITY;
+                for (int r = 0; r < 16; r++) {
+                    const int back = qp - (kp + j * 32 + (r >> 2) * 8 + half * 4 + (r & 3));
+                    s[j][r] = (unsigned)back < (unsigned)far ? s[j][r] * sc2 : -INFINITY;
+                    mx = fmaxf(mx, s[j][r]);
                 }
-                s[j][r] = v;
-                mx = fmaxf(mx, v);
-            }
+        } else {
+#pragma unroll
+            for (int j = 0; j < 2; j++)
+#pragma unroll
+                for (int r = 0; r < 16; r++) {
+                    s[j][r] *= sc2;
+                    mx = fmaxf(mx, s[j][r]);
+                }
+        }
         mx = fmaxf(mx, lane_xor_f<32>(mx));
         const float al = __builtin_amdgcn_exp2f(m - mx);
         m = mx;
@@ -528,10 +647,16 @@ int latent_flash(const LatentDims& d, const bf16_t* q, int ldq, const bf16_t* k,
                  int kv0, int pos0, int tokens, bf16_t* o, int ldo, hipStream_t st) {
     const int rows = pos0 + tokens - kv0;
     FX_REQUIRE(q && k && vt && cache && o && tokens > 0 && latent_flash_ok(d), "latent_flash: dim=%d rot=%d vdim=%d", d.dim, d.rot_dim, d.vdim);
+    FX_REQUIRE((size_t)rows * ldk < (1ull << 31) && (size_t)rows * d.ldc < (1ull << 31) && (size_t)d.vdim * ldv < (1ull << 31), "latent_flash: %d rows", rows);
     FX_REQUIRE(ldq % 8 == 0 && ldk % 8 == 0 && ldv % 64 == 0 && ldv >= rows && ldo % 4 == 0 && kv0 >= 0 && pos0 >= kv0 && pos0 + tokens <= d.capacity,
                "latent_flash: strides %d %d %d %d, rows %d", ldq, ldk, ldv, ldo, rows);
-    const int grid = (tokens + kFlashQ - 1) / kFlashQ * d.heads, dk = flash_dk(d), dv = d.vdim;
-#define FX_FLASH(DK, DV) latent_flash_kernel<DK, DV><<<grid, 256, 0, st>>>(d, q, ldq, k, ldk, vt, ldv, cache, kv0, pos0, tokens, rows, o, ldo)
+    const int dk = flash_dk(d), dv = d.vdim, g4 = (tokens + 127) / 128 * d.heads, g2 = (tokens + 63) / 64 * d.heads;
+    // two waves per workgroup where four would leave CUs without one
+#define FX_FLASH(DK, DV)                                                                                                                   \
+    do {                                                                                                                                   \
+        if (g4 >= 256) latent_flash_kernel<DK, DV, 4><<<g4, 256, 0, st>>>(d, q, ldq, k, ldk, vt, ldv, cache, kv0, pos0, tokens, rows, o, ldo); \
+        else latent_flash_kernel<DK, DV, 2><<<g2, 128, 0, st>>>(d, q, ldq, k, ldk, vt, ldv, cache, kv0, pos0, tokens, rows, o, ldo);         \
+    } while (0)
     if (dk <= 64 && dv <= 64) FX_FLASH(64, 64);
     else if (dk <= 128 && dv <= 64) FX_FLASH(128, 64);
     else if (dk <= 128 && dv <= 128) FX_FLASH(128, 128);
