@@ -10,38 +10,36 @@ namespace fx {
 constexpr int kMaxExperts = 1024, kMaxTop = 32;
 
 // Expert choice of one token by one wave: softmax over the router outputs, the `top` largest (ties: lower index), their
-// weights divided by their sum.  sel / wt: LDS, filled by every lane's agreement (lane 0 writes).
-__device__ __forceinline__ void route_wave(const float* __restrict__ z, int experts, int top, int* sel, float* wt) {
+// weights divided by their sum.  Lane k < top gets choice k and its weight.  NE: 64-expert pieces (experts <= 64 NE).
+template <int NE>
+__device__ __forceinline__ void route_wave_n(const float* __restrict__ z, int experts, int top, int& pick, float& weight) {
     const int lane = threadIdx.x & 63;
-    float v[kMaxExperts / 64];
+    float v[NE];
     float mx = -INFINITY;
 #pragma unroll
-    for (int i = 0; i < kMaxExperts / 64; i++) {
-        const int e = i * 64 + lane;
-        v[i] = -INFINITY;
-        if (i * 64 < experts && e < experts) v[i] = z[e];
+    for (int i = 0; i < NE; i++) {
+        v[i] = i * 64 + lane < experts ? z[i * 64 + lane] : -INFINITY;
         mx = fmaxf(mx, v[i]);
     }
     mx = wave_max(mx);
     float den = 0.0f;
 #pragma unroll
-    for (int i = 0; i < kMaxExperts / 64; i++) {
-        if (i * 64 >= experts) continue;
-        v[i] = i * 64 + lane < experts ? exp_f(v[i] - mx) : -1.0f;
+    for (int i = 0; i < NE; i++) {
+        v[i] = i * 64 + lane < experts ? exp_f<false>(v[i] - mx) : -1.0f;
         den += fmaxf(v[i], 0.0f);
     }
     den = wave_sum(den);
     float sum = 0.0f;
+    pick = 0;
+    weight = 0.0f;
     for (int k = 0; k < top; k++) {
-        float best = -2.0f;
+        float best = v[0];
 #pragma unroll
-        for (int i = 0; i < kMaxExperts / 64; i++)
-            if (i * 64 < experts) best = fmaxf(best, v[i]);
+        for (int i = 1; i < NE; i++) best = fmaxf(best, v[i]);
         best = wave_max(best);
         int bi = -1;                                      // lowest index that holds the maximum
 #pragma unroll
-        for (int i = 0; i < kMaxExperts / 64; i++) {
-            if (i * 64 >= experts) continue;
+        for (int i = 0; i < NE; i++) {
             const unsigned long long hit = __ballot(v[i] == best);
             if (bi < 0 && hit) {
                 const int l = __builtin_ctzll(hit);
@@ -51,10 +49,14 @@ __device__ __forceinline__ void route_wave(const float* __restrict__ z, int expe
         }
         const float s = best / den;
         sum += s;
-        if (lane == 0) { sel[k] = bi; wt[k] = s; }
+        if (lane == k) { pick = bi; weight = s; }
     }
-    if (lane == 0)
-        for (int k = 0; k < top; k++) wt[k] = wt[k] / (sum + 1e-20f);
+    weight = weight / (sum + 1e-20f);
+}
+__device__ __forceinline__ void route_wave(const float* __restrict__ z, int experts, int top, int& pick, float& weight) {
+    if (experts <= 64) route_wave_n<1>(z, experts, top, pick, weight);
+    else if (experts <= 256) route_wave_n<4>(z, experts, top, pick, weight);
+    else route_wave_n<kMaxExperts / 64>(z, experts, top, pick, weight);
 }
 
 // VEC: the prologue keeps its vectors in registers as float4 (k a multiple of 4, at most what the S pieces per thread cover);
@@ -65,8 +67,6 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     extern __shared__ __attribute__((aligned(16))) float xs[];     // [kpad] the vector
     __shared__ float red[2][4 * R];
     __shared__ float nred[4];
-    __shared__ int sel[kMaxTop];
-    __shared__ float wt[kMaxTop];
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
     const int tok = PRO == 2 ? blockIdx.y / g.top : blockIdx.y;
     const ET* w = static_cast<const ET*>(g.w);
@@ -93,11 +93,12 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
         __builtin_amdgcn_sched_barrier(0);
     }
     if constexpr (PRO == 2) {
-        if (wave == 0) route_wave(g.route + (size_t)tok * g.ld_route, g.experts, g.top, sel, wt);
-        __syncthreads();
+        int pick;                                         // every wave chooses for itself: no barrier before the weights
+        float weight;
+        route_wave(g.route + (size_t)tok * g.ld_route, g.experts, g.top, pick, weight);
         const int slot = blockIdx.y % g.top;
-        w += (size_t)__builtin_amdgcn_readfirstlane(sel[slot]) * g.w_stride;
-        if (blockIdx.x == 0 && t == 0) { g.pick[blockIdx.y] = sel[slot]; g.pick_w[blockIdx.y] = wt[slot]; }
+        w += (size_t)__builtin_amdgcn_readlane(pick, slot) * g.w_stride;
+        if (blockIdx.x == 0 && t == slot) { g.pick[blockIdx.y] = pick; g.pick_w[blockIdx.y] = weight; }
     }
     const int nchunk = g.kpad / CE;                       // 16-byte pieces of a row
     const int ng = (g.n + R - 1) / R, G = gridDim.x;      // groups of R rows, dealt to the workgroups in turn
@@ -326,28 +327,24 @@ template int moe_down_small<float>(const MoeDownArgs&, int, hipStream_t);
 static __global__ __launch_bounds__(256) void moe_clear_kernel(int* counts, int n) {
     for (int i = threadIdx.x; i < n; i += 256) counts[i] = 0;
 }
-constexpr int kPlanT = 1024, kRouteRows = 64;              // rows per workgroup of the route kernel
+constexpr int kPlanT = 1024, kRouteRows = 32;              // rows per workgroup of the route kernel
 static __global__ __launch_bounds__(kPlanT) void moe_route_kernel(const float* __restrict__ route, int ld, int rows, int experts, int top,
                                                                   int* __restrict__ pick, float* __restrict__ pick_w, int* __restrict__ counts) {
-    __shared__ int sel[kPlanT / 64][kMaxTop], hist[kMaxExperts];
-    __shared__ float wt[kPlanT / 64][kMaxTop];
+    __shared__ int hist[kMaxExperts];
     const int t = threadIdx.x, wave = t >> 6, lane = t & 63;
     for (int e = t; e < experts; e += kPlanT) hist[e] = 0;
     __syncthreads();
     for (int i = 0; i < kRouteRows / (kPlanT / 64); i++) {
         const int row = blockIdx.x * kRouteRows + i * (kPlanT / 64) + wave;
         if (row >= rows) break;
-        route_wave(route + (size_t)row * ld, experts, top, sel[wave], wt[wave]);
-        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-        __builtin_amdgcn_wave_barrier();
+        int e;
+        float w;
+        route_wave(route + (size_t)row * ld, experts, top, e, w);
         if (lane < top) {
-            const int e = sel[wave][lane];
             pick[row * top + lane] = e;
-            pick_w[row * top + lane] = wt[wave][lane];
+            pick_w[row * top + lane] = w;
             atomicAdd(&hist[e], 1);
         }
-        __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-        __builtin_amdgcn_wave_barrier();
     }
     __syncthreads();
     for (int e = t; e < experts; e += kPlanT)

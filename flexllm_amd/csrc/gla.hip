@@ -87,32 +87,31 @@ __global__ __launch_bounds__(kGlaStepT) void gla_step_kernel(GlaDims d, const PT
     }
 }
 
-// The same with the head's state in registers: 1024 threads, thread (g, c) holds rows g, g + groups, ... of column c.
+// The same with the head's state in registers: 1024 threads, thread (g, c) holds a run of rows of column c.
 // Everything that does not depend on the token's decay is requested at the start, in one trip to memory.
 constexpr int kGlaRegT = 1024, kGlaRegRows = 16, kGlaRegRank = 16;
 static bool gla_regs_ok(const GlaDims& d) {
     return d.vdim <= 512 && d.dim <= kGlaRegT && d.dim <= kGlaRegT / d.vdim * kGlaRegRows && d.a_rank <= 1024;
 }
+static __host__ __device__ int gla_reg_rows(int dim, int groups) { return ((dim + groups - 1) / groups + 3) / 4 * 4; }   // <= kGlaRegRows
 template <typename ET, typename PT, typename OT>
 __global__ __launch_bounds__(kGlaRegT) void gla_step_regs_kernel(GlaDims d, const PT* __restrict__ p, int ldp, const float* __restrict__ a1, int ld_a1,
                                                                  const ET* __restrict__ w_a2, const float* __restrict__ b_a2,
                                                                  const float* __restrict__ norm_w, float* __restrict__ state,
                                                                  const int* __restrict__ pos_state, int tok0, int tokens, OT* __restrict__ o, int ldo) {
     constexpr int CE = Chunk<ET>::N, NW = kGlaRegRank / CE;
-    extern __shared__ float sm[];                         // q, k, decay [dim]; gate input [rank]; sums [groups][vdim]
+    extern __shared__ __attribute__((aligned(16))) float sm[];     // q, k, decay [dim, padded]; gate input [rank]; sums [groups][vdim]
     __shared__ float red[kGlaRegT / 64];
     const int t = threadIdx.x, h = blockIdx.x, HD = d.heads * d.dim, HV = d.heads * d.vdim, lda2 = pad_k(d.a_rank);
-    float *sq = sm, *sk = sq + d.dim, *sa = sk + d.dim, *s1 = sa + d.dim, *sum = s1 + d.a_rank;
-    const int groups = kGlaRegT / d.vdim, c = t % d.vdim, g = t / d.vdim;
+    const int groups = kGlaRegT / d.vdim, c = t % d.vdim, g = t / d.vdim, rows = gla_reg_rows(d.dim, groups), dp = groups * rows, i0 = g * rows;
+    float *sq = sm, *sk = sq + dp, *sa = sk + dp, *s1 = sa + dp, *sum = s1 + d.a_rank;
     const bool mine = g < groups, row_t = t < d.dim, col_t = t < d.vdim;
     float* S = state + (size_t)h * d.dim * d.vdim;
     const int pos = pos_state[0] + tok0;
     float s[kGlaRegRows];
 #pragma unroll
-    for (int j = 0; j < kGlaRegRows; j++) {
-        const int i = g + j * groups;
-        s[j] = mine && i < d.dim ? S[(size_t)i * d.vdim + c] : 0.0f;
-    }
+    for (int j = 0; j < kGlaRegRows; j++) s[j] = mine && j < rows && i0 + j < d.dim ? S[(size_t)(i0 + j) * d.vdim + c] : 0.0f;
+    for (int i = d.dim + t; i < dp; i += kGlaRegT) { sq[i] = 0.0f; sk[i] = 0.0f; sa[i] = 0.0f; }
     uint4 w[NW];
     const int ch = h * d.dim + t;
 #pragma unroll
@@ -144,14 +143,18 @@ __global__ __launch_bounds__(kGlaRegT) void gla_step_regs_kernel(GlaDims d, cons
         __syncthreads();
         const bool fresh = pos + n == 0;                  // a sequence starts from a zero state
         float acc = 0.0f;
+        if (mine)
 #pragma unroll
-        for (int j = 0; j < kGlaRegRows; j++) {
-            const int i = g + j * groups;
-            if (mine && i < d.dim) {
-                s[j] = fma_f(sk[i], v, fresh ? 0.0f : s[j] * sa[i]);
-                acc = fma_f(s[j], sq[i], acc);
+            for (int j = 0; j < kGlaRegRows; j += 4) {
+                if (j >= rows) break;
+                const f32x4 k4 = *reinterpret_cast<const f32x4*>(sk + i0 + j), a4 = *reinterpret_cast<const f32x4*>(sa + i0 + j),
+                            q4 = *reinterpret_cast<const f32x4*>(sq + i0 + j);
+#pragma unroll
+                for (int e = 0; e < 4; e++) {
+                    s[j + e] = fma_f(k4[e], v, fresh ? 0.0f : s[j + e] * a4[e]);
+                    acc = fma_f(s[j + e], q4[e], acc);
+                }
             }
-        }
         if (mine) sum[g * d.vdim + c] = acc;
         __syncthreads();
         float x = 0.0f;
@@ -161,10 +164,8 @@ __global__ __launch_bounds__(kGlaRegT) void gla_step_regs_kernel(GlaDims d, cons
         if (col_t) o[(size_t)(tok0 + n) * ldo + h * d.vdim + t] = (OT)(x * rs * nw * (gate * sigmoid_f(gate)));
     }
 #pragma unroll
-    for (int j = 0; j < kGlaRegRows; j++) {
-        const int i = g + j * groups;
-        if (mine && i < d.dim) S[(size_t)i * d.vdim + c] = s[j];
-    }
+    for (int j = 0; j < kGlaRegRows; j++)
+        if (mine && j < rows && i0 + j < d.dim) S[(size_t)(i0 + j) * d.vdim + c] = s[j];
 }
 
 template <typename ET>
@@ -172,7 +173,8 @@ int gla_steps(const GlaDims& d, const void* p, int ldp, int p_f32, const float* 
               const float* norm_w, float* state, const int* pos_state, int tok0, int tokens, void* o, int ldo, int o_f32, hipStream_t st) {
     FX_REQUIRE(p && a1 && w_a2 && b_a2 && norm_w && state && pos_state && o && tokens > 0, "gla_steps: null pointer");
     if (gla_regs_ok(d)) {
-        const size_t lds = sizeof(float) * (3 * d.dim + d.a_rank + (size_t)(kGlaRegT / d.vdim) * d.vdim);
+        const int groups = kGlaRegT / d.vdim;
+        const size_t lds = sizeof(float) * (3 * (size_t)groups * gla_reg_rows(d.dim, groups) + d.a_rank + (size_t)groups * d.vdim);
 #define FX_GLA(PT, OT) gla_step_regs_kernel<ET, PT, OT><<<d.heads, kGlaRegT, lds, st>>>(d, static_cast<const PT*>(p), ldp, a1, ld_a1, w_a2, b_a2, norm_w, state, pos_state, tok0, tokens, static_cast<OT*>(o), ldo)
         FX_REQUIRE((p_f32 != 0) == (o_f32 != 0), "gla_steps: input and output are both float32 or both of the element type");
         if (p_f32) FX_GLA(float, float);
@@ -207,14 +209,17 @@ size_t gla_chunk_scratch(const GlaDims& d, int tokens) {
 
 constexpr float kGlaMild = -40.0f;                        // smallest running sum for which e^{-L} is formed
 
-// Running sums of log decay inside each chunk, cum [tokens][heads * dim].
-template <typename ET, int RMAX>
+// Running sums of log decay inside each chunk, cum [tokens][heads * dim].  64 channels per workgroup; a wave takes a quarter
+// of the chunk's tokens and adds the earlier quarters' totals at the end.
+template <typename ET, int RMAX, int C>
 __global__ __launch_bounds__(256) void gla_cum_kernel(GlaDims d, const float* __restrict__ a1, int ld_a1, const ET* __restrict__ w_a2,
-                                                      const float* __restrict__ b_a2, int tokens, int C, float* __restrict__ cum) {
+                                                      const float* __restrict__ b_a2, int tokens, float* __restrict__ cum) {
     constexpr bool kRegs = RMAX > 0;
+    constexpr int Q = C / 4;
     const int rp = kRegs ? RMAX : d.a_rank;               // row length in LDS, zero beyond the rank
     extern __shared__ __attribute__((aligned(16))) float s1[];
-    const int t = threadIdx.x, tok0 = blockIdx.x * C, n = min(C, tokens - tok0), HD = d.heads * d.dim, ch = blockIdx.y * 256 + t;
+    __shared__ float total[4][64];
+    const int t = threadIdx.x, tok0 = blockIdx.x * C, n = min(C, tokens - tok0), HD = d.heads * d.dim, ch = blockIdx.y * 64 + (t & 63), q = t >> 6;
     for (int i = t; i < n * rp; i += 256) {
         const int r = i / rp, c = i - r * rp;
         s1[i] = c < d.a_rank ? a1[(size_t)(tok0 + r) * ld_a1 + c] : 0.0f;
@@ -233,10 +238,10 @@ __global__ __launch_bounds__(256) void gla_cum_kernel(GlaDims d, const float* __
         }
     }
     __syncthreads();
-    if (ch >= HD) return;
-    float s = 0.0f;
-#pragma unroll 4
-    for (int i = 0; i < n; i++) {
+    float run[Q], s = 0.0f;
+#pragma unroll
+    for (int j = 0; j < Q; j++) {
+        const int i = min(q * Q + j, n - 1);
         float z = b;
         if constexpr (kRegs) {
 #pragma unroll
@@ -249,8 +254,16 @@ __global__ __launch_bounds__(256) void gla_cum_kernel(GlaDims d, const float* __
             for (int r = 0; r < d.a_rank; r++) z = fma_f((float)w[r], s1[i * d.a_rank + r], z);
         }
         s += log_sigmoid_f(z) * inv;
-        cum[(size_t)(tok0 + i) * HD + ch] = s;
+        run[j] = s;
     }
+    total[q][t & 63] = s;
+    __syncthreads();
+    float before = 0.0f;
+    for (int i = 0; i < q; i++) before += total[i][t & 63];
+    if (ch >= HD) return;
+#pragma unroll
+    for (int j = 0; j < Q; j++)
+        if (q * Q + j < n) cum[(size_t)(tok0 + q * Q + j) * HD + ch] = run[j] + before;
 }
 
 // Contribution of a chunk to the state behind it, U [dim][vdim], the chunk's whole decay, and whether the decay is mild.
@@ -687,11 +700,11 @@ static int gla_chunks_c(const GlaDims& d, const ET* p, int ldp, const float* a1,
     int* mild = reinterpret_cast<int*>(cum + (size_t)nc * C * HD);
     int rc;
     {
-        const dim3 grid(nc, (HD + 255) / 256);
+        const dim3 grid(nc, (HD + 63) / 64);
         const size_t lds = sizeof(float) * C * (d.a_rank <= 16 ? 16 : d.a_rank <= 32 ? 32 : d.a_rank);
-        if (d.a_rank <= 16) gla_cum_kernel<ET, 16><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, C, cum);
-        else if (d.a_rank <= 32) gla_cum_kernel<ET, 32><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, C, cum);
-        else gla_cum_kernel<ET, 0><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, C, cum);
+        if (d.a_rank <= 16) gla_cum_kernel<ET, 16, C><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, cum);
+        else if (d.a_rank <= 32) gla_cum_kernel<ET, 32, C><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, cum);
+        else gla_cum_kernel<ET, 0, C><<<grid, 256, lds, st>>>(d, a1, ld_a1, w_a2, b_a2, tokens, cum);
     }
     const int walk = (int)(((size_t)HD * d.vdim + 255) / 256);
     bool vec = false;

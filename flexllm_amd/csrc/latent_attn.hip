@@ -269,7 +269,6 @@ __global__ __launch_bounds__(256) void latent_split_tile_kernel(LatentDims d, co
     float *sc = sq + d.ldc, *sum = sc + tk;
     const float* qv = ql + ((size_t)tok * d.heads + h) * d.ldc;
     const int pos = state[0] + tok0 + tok;
-    for (int i = t; i < d.ldc; i += 256) sq[i] = qv[i];
     const int lo = d.window > 0 && pos - d.window + 1 > 0 ? pos - d.window + 1 : 0;
     const int first = lo + blockIdx.x * keys, n = min(keys, pos + 1 - first);
     if (n <= 0 || pos >= d.capacity) return;
@@ -281,11 +280,13 @@ __global__ __launch_bounds__(256) void latent_split_tile_kernel(LatentDims d, co
         const int nk = min(tk, n - k0), total = nk * nch;
         const i32x4* src = reinterpret_cast<const i32x4*>(cache + (size_t)(first + k0) * d.ldc);    // the rows are one run of memory
         i32x4* dst = reinterpret_cast<i32x4*>(rows);
-        __syncthreads();                                  // the previous tile has been read; q is in
+        __syncthreads();                                  // the previous tile has been read
         for (int b = 0; b < total; b += 256 * kSplitPieces) {
             i32x4 u[kSplitPieces];
 #pragma unroll
             for (int i = 0; i < kSplitPieces; i++) u[i] = src[min(b + 256 * i + t, total - 1)];
+            if (k0 == 0 && b == 0)                        // the query follows the first rows on their way
+                for (int i = t; i < d.ldc; i += 256) sq[i] = qv[i];
 #pragma unroll
             for (int i = 0; i < kSplitPieces; i++)
                 if (b + 256 * i + t < total) dst[b + 256 * i + t] = u[i];
