@@ -424,7 +424,7 @@ def nifunex_main(args):
     from flexllm_amd.device import Event
     res = {"metric": "Nifunex decode tok/s + prefill ms", "dtype": "bf16", "data": "synthetic", "device": fx.device.device_name(), "sizes": {}}
     for name in args.nifunex.split(","):
-        res["sizes"][name] = nifunex_leg(name, args.steps, args.warmup)
+        res["sizes"][name] = nifunex_leg(name, args.steps, args.warmup, tuple(int(n) for n in args.nifunex_prompts.split(",")))
     if not args.no_prefill:
         cfg = llama.make_config()
         model = llama.Llama(cfg, llama.synth_weights(cfg, seed=1, device=True, embed_range=0.03))
@@ -468,6 +468,7 @@ def main():
     ap.add_argument("--nifunex", nargs="?", const="1b-dense,1b-moe,8b-dense", default=None, metavar="SIZES",
                     help="only run the Nifunex sizes (1b-dense, 1b-moe, 8b-dense; all when none is named) and, unless --no-prefill, "
                          "Llama-3.2-1B W8A8 beside them")
+    ap.add_argument("--nifunex-prompts", default="1024,4096", help="prompt lengths of the --nifunex legs; decoding starts behind the longest")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on one GPU only (no collectives, no sharding); use --gpus 1", file=sys.stderr)

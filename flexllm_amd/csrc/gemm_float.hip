@@ -377,3 +377,18 @@ template int gemm_grouped<bf16_t>(const GemmArgs&, int, hipStream_t);
 template int gemm_grouped<float>(const GemmArgs&, int, hipStream_t);
 
 }  // namespace fx
+
+using namespace fx;
+
+extern "C" {
+
+int flexllm_linear_float_gemm(const void* a, const void* w, void* y, float* y32, int m, int k, int n, int n_split, int glu, float limit,
+                              int dtype, void* stream) {
+    FX_REQUIRE(dtype == 0 || dtype == 1, "linear_float_gemm: dtype=%d", dtype);
+    GemmArgs g;
+    g.a = a; g.w = w; g.lda = k; g.m = m; g.n = n; g.k = k; g.n_split = n_split; g.glu = glu; g.limit = limit;
+    g.y = y; g.ldy = glu ? n_split / 2 : n_split; g.y32 = y32; g.ldy32 = n - n_split;
+    return dtype == 0 ? gemm_float<bf16_t>(g, as_stream(stream)) : gemm_float<float>(g, as_stream(stream));
+}
+
+}  // extern "C"

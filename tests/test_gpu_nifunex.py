@@ -55,6 +55,8 @@ ALONE = {
     "gla one head, wide values": nc.config([nc.gla(heads=1, dim=16, vdim=96, tau=1.0)]),
     "gla beyond one chunk size": nc.config([nc.gla(heads=2, dim=144, vdim=136)]),
     "gla beyond the chunk kernels": nc.config([nc.gla(heads=1, dim=264, vdim=24)]),
+    "gla, 72 channels": nc.config([nc.gla(heads=2, dim=72, vdim=128)]),
+    "gla, 128 channels": nc.config([nc.gla(heads=1, dim=128, vdim=88, tau=16.0)]),
     "latent": nc.config([nc.latent()]),
     "latent without window": nc.config([nc.latent(window=None)]),
     "latent without yarn": nc.config([nc.latent(scaling=None)]),
@@ -64,6 +66,9 @@ ALONE = {
     "latent, wide values": nc.config([nc.latent(heads=1, dim=64, rot_dim=32, vdim=160, kv_rank=96)]),
     "latent, odd sizes": nc.config([nc.latent(heads=3, dim=10, rot_dim=6, vdim=7, kv_rank=30)]),
     "latent, other layer's rows": nc.config([nc.latent(window=20), nc.latent(heads=2, dim=8, vdim=16, window=50, scale=0.4, kv_from=0)]),
+    "latent, long rows": nc.config([nc.latent(heads=1, dim=16, vdim=16, kv_rank=2100)]),
+    "dense, vectors of some length": nc.config([nc.gla(mlp=nc.dense(ff=3000))], width=64),
+    "dense, long vectors": nc.config([nc.gla(mlp=nc.dense(ff=8300))], width=64),
     "dense": nc.config([nc.gla(mlp=nc.dense(ff=100, limit=0.5))]),
     "mixture": nc.config([nc.gla(mlp=nc.moe(shared=0))]),
     "mixture, top 1": nc.config([nc.gla(mlp=nc.moe(experts=9, top=1, shared=0))]),
@@ -231,6 +236,41 @@ def test_slots(dtype):
     for n, g in (("a", got_a), ("b", got_b), ("c", got_c)):
         close(np.concatenate(g), want[n], dtype, n)
     m.close()
+
+
+@BOTH
+def test_many_visible_keys(dtype):
+    """More keys than one tile per split holds, so that the splits' running maxima come into play."""
+    cfg = nc.config([nc.latent(heads=1, dim=16, rot_dim=8, vdim=16, kv_rank=512, window=None, scale=0.5)], width=96, vocab=90)
+    w, toks = nc.weights(cfg, 19), nc.tokens(cfg, 2310)
+    want = expect(cfg, w, toks)
+    m = model(cfg, w, dtype, max_pos=2600)
+    slot = m.pool.acquire(0)
+    m.step(slot, toks[:2300])
+    got = [m.step(slot, toks[2300 + i:2301 + i], [0]) for i in range(10)]
+    close(np.concatenate(got), want[2300:], dtype)
+    m.close()
+
+
+@BOTH
+@pytest.mark.parametrize("m,k,n,split,glu", [(1024, 64, 16384, 16384, 1), (1024, 128, 4096, 4096, 0), (1000, 192, 3648, 3072, 0), (300, 64, 272, 256, 0),
+                                             (64, 256, 2048, 0, 0), (9, 64, 37, 22, 1), (130, 64, 301, 150, 0), (2048, 64, 2112, 2048, 1)])
+def test_gemm(m, k, n, split, glu, dtype):
+    """Every tile shape of the GEMM, ragged sizes, the split between the two outputs, the gated unit in the epilogue."""
+    from flexllm_amd import ops, to_device
+    from flexllm_amd.loader import from_bf16, to_bf16
+    r = np.random.default_rng(m + n)
+    a, w = [from_bf16(to_bf16(r.standard_normal(s).astype(np.float32))) for s in ((m, k), (n, k))]
+    dev = to_device if dtype == "float32" else lambda x: to_device(to_bf16(x))
+    y, y32 = ops.linear_float(dev(a), dev(w), split, bool(glu), 3.0)
+    want = a.astype(np.float64) @ w.astype(np.float64).T
+    if split:
+        first = nifunex_ref.clamped_glu(want[:, 0:split:2], want[:, 1:split:2], 3.0) if glu else want[:, :split]
+        got = y.numpy() if dtype == "float32" else from_bf16(y.numpy())
+        tol = 1e-5 if dtype == "float32" else 5e-3
+        assert np.all(np.abs(got - first) <= tol * (np.abs(first) + np.sqrt(k)))
+    if split < n:
+        assert np.all(np.abs(y32.numpy() - want[:, split:]) <= 1e-5 * (np.abs(want[:, split:]) + np.sqrt(k)))
 
 
 def test_first_tokens():
