@@ -42,7 +42,9 @@ class LlamaW4A4Weights(C.Structure):
 
 
 class HybridConfig(C.Structure):
-    _fields_ = [(n, C.c_int) for n in ("layers", "width", "vocab", "max_pos", "slots", "dtype")] + [("eps", C.c_float)]
+    _fields_ = [(n, C.c_int) for n in ("layers", "width", "vocab", "max_pos", "slots", "dtype")] + \
+               [(n, C.c_float) for n in ("eps", "embed_scale", "norm_add")] + \
+               [(n, C.c_int) for n in ("post_norms", "loop_start", "loop_stop", "loop_times")]
 
 
 class HybridLayer(C.Structure):
@@ -50,6 +52,7 @@ class HybridLayer(C.Structure):
                [("scale", C.c_float)] + \
                [(n, C.c_double) for n in ("rot_base", "yarn_factor", "yarn_original", "yarn_fast", "yarn_slow")] + \
                [("a_rank", C.c_int), ("tau", C.c_float)] + \
+               [(n, C.c_int) for n in ("kv_heads", "sink", "temp_every")] + [("temp_coef", C.c_float), ("glu", C.c_int)] + \
                [(n, C.c_int) for n in ("ff_kind", "ff", "experts", "top", "shared_ff")] + \
                [("limit", C.c_float), ("shared_limit", C.c_float)]
 
@@ -57,7 +60,7 @@ class HybridLayer(C.Structure):
 class HybridLayerWeights(C.Structure):
     _fields_ = [(n, C.c_void_p) for n in
                 ("norm1", "norm1b", "norm2", "norm2b", "q", "o", "dkv", "dkv_norm", "uk", "uv",
-                 "k", "v", "g", "a1", "a2", "a2_bias", "head_norm", "gate", "up", "down",
+                 "k", "v", "g", "a1", "a2", "a2_bias", "head_norm", "q_bias", "k_bias", "q_norm", "k_norm", "gate", "up", "down",
                  "router", "shared_gate", "shared_up", "shared_down", "shared_sg", "expert_gate", "expert_up", "expert_down")]
 
 

@@ -25,7 +25,7 @@ def sources():
 
 # Parts of the library that can be built and loaded on their own (a checkout without built files then compiles what one
 # model needs and nothing else).
-COMPONENTS = {"hybrid": ("runtime", "hybrid", "gemm_float", "gemv_float", "rows_float", "latent_attn", "gla")}
+COMPONENTS = {"hybrid": ("runtime", "hybrid", "gemm_float", "gemv_float", "rows_float", "latent_attn", "shared_kv_attn", "gla")}
 
 
 def component(name):

@@ -46,6 +46,18 @@ __device__ __forceinline__ float clamped_glu_f(float gate, float up, float limit
     return g * sigmoid_f(1.702f * g) * (u + 1.0f);
 }
 
+// Gated linear unit with the tanh form of gelu: 0.5 z (1 + tanh(u)) = z sigmoid(2u), u = sqrt(2/pi) (z + 0.044715 z^3)
+__device__ __forceinline__ float gelu_glu_f(float gate, float up) {
+    const float u = 0.7978845608028654f * fma_f(0.044715f * gate * gate, gate, gate);
+    return gate * sigmoid_f(2.0f * u) * up;
+}
+
+// The units that the linears can apply to gate/up pairs (GemmArgs::glu, GemvArgs::glu; 0: none)
+enum GluKind { kGluClamped = 1, kGluGelu = 2 };
+__device__ __forceinline__ float glu_f(int kind, float gate, float up, float limit) {
+    return kind == kGluGelu ? gelu_glu_f(gate, up) : clamped_glu_f(gate, up, limit);
+}
+
 // R sums over the 64 lanes of a wave at once: every halving step hands half of the values to the partner lane, so the
 // total is 2R moves instead of 6R.  Afterwards lane l (l < R) holds the sum of row multi_row<R>(l).
 template <int R, int MASK>

@@ -3,7 +3,7 @@
 // bfloat16: the direct-load kernel of the int8 path (gemm_i8.h) on v_mfma_f32_32x32x16_bf16.  A lane's operand is the
 // same 16 bytes of a row as in the int8 instruction, so the LDS stage layout, the chunk rotation and the software
 // pipeline carry over with K counted in bytes.  Additions: rows of A may be gathered, groups of rows may have a weight
-// matrix each (experts), the epilogue splits the columns between an ET and a float32 output and applies the clamped
+// matrix each (experts), the epilogue adds a bias, splits the columns between an ET and a float32 output and applies the
 // gated unit to interleaved gate/up columns.
 //
 // float32: v_mfma_f32_32x32x2_f32 (full float32 products and sums) on register-staged 64x64 tiles, same epilogue.
@@ -39,16 +39,20 @@ __device__ __forceinline__ bool gemm_pick_tile(const GemmArgs& g, int tiles_m, i
 
 // One row's four consecutive columns col..col+3 of the accumulator tile.
 template <typename ET>
-__device__ __forceinline__ void gemm_store4(const GemmArgs& g, int row, int col, const float (&v)[4], bool vec) {
+__device__ __forceinline__ void gemm_store4(const GemmArgs& g, int row, int col, float (&v)[4], bool vec) {
     ET* y = static_cast<ET*>(g.y);
+    if (g.bias) {
+#pragma unroll
+        for (int e = 0; e < 4; e++) v[e] += g.bias[min(col + e, g.n - 1)];
+    }
     if (vec) {
         if (col >= g.n) return;
         if (col >= g.n_split) {
             *reinterpret_cast<float4*>(g.y32 + (size_t)row * g.ldy32 + (col - g.n_split)) = make_float4(v[0], v[1], v[2], v[3]);
         } else if (g.glu) {
             ET* d = y + (size_t)row * g.ldy + (col >> 1);
-            d[0] = (ET)clamped_glu_f(v[0], v[1], g.limit);
-            d[1] = (ET)clamped_glu_f(v[2], v[3], g.limit);
+            d[0] = (ET)glu_f(g.glu, v[0], v[1], g.limit);
+            d[1] = (ET)glu_f(g.glu, v[2], v[3], g.limit);
         } else if constexpr (std::is_same<ET, float>::value) {
             *reinterpret_cast<float4*>(y + (size_t)row * g.ldy + col) = make_float4(v[0], v[1], v[2], v[3]);
         } else {
@@ -65,7 +69,7 @@ __device__ __forceinline__ void gemm_store4(const GemmArgs& g, int row, int col,
         if (c >= g.n) return;
         if (c >= g.n_split) g.y32[(size_t)row * g.ldy32 + (c - g.n_split)] = v[e];
         else if (!g.glu) y[(size_t)row * g.ldy + c] = (ET)v[e];
-        else if ((c & 1) == 0) y[(size_t)row * g.ldy + (c >> 1)] = (ET)clamped_glu_f(v[e], v[(e + 1) & 3], g.limit);
+        else if ((c & 1) == 0) y[(size_t)row * g.ldy + (c >> 1)] = (ET)glu_f(g.glu, v[e], v[(e + 1) & 3], g.limit);
     }
 }
 
@@ -90,7 +94,7 @@ __device__ __forceinline__ void gemm_epilogue(const GemmArgs& g, const GemmTile&
             for (int p = 0; p < 4; p++) {
                 const int lr = p * 8 + pr, row = t.row0 + wm + i * 32 + lr;
                 const f32x4 q = *reinterpret_cast<const f32x4*>(patch + lr * EP + pc);
-                const float v[4] = {q[0], q[1], q[2], q[3]};
+                float v[4] = {q[0], q[1], q[2], q[3]};
                 if (row < t.row_end) gemm_store4<ET>(g, row, col0 + wn + j * 32 + pc, v, vec);
             }
             __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
@@ -261,7 +265,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_narrow_kernel(GemmArgs g, int n
     __syncthreads();
     const int rr = t >> 4, cc = t & 15;
     const float v = (part[0][rr * 17 + cc] + part[1][rr * 17 + cc]) + (part[2][rr * 17 + cc] + part[3][rr * 17 + cc]);
-    if (row0 + rr < g.m && col0 + cc < g.n) g.y32[(size_t)(row0 + rr) * g.ldy32 + (col0 + cc - g.n_split)] = v;
+    if (row0 + rr < g.m && col0 + cc < g.n) g.y32[(size_t)(row0 + rr) * g.ldy32 + (col0 + cc - g.n_split)] = g.bias ? v + g.bias[col0 + cc] : v;
 }
 
 int gemm_group_tile_rows(int rows_per_group) { return rows_per_group >= 96 ? 128 : 64; }

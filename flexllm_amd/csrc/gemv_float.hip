@@ -75,7 +75,9 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     constexpr int Q = VEC ? S * CE / 4 : 1;               // float4 per thread
     f32x4 xv[Q], yv[Q], gb[Q], gv[Q];
     const int k4 = g.k >> 2;
-    const bool have_y = PRO == 1 && g.y != nullptr;
+    const bool have_y = PRO == 1 && g.y != nullptr, post = have_y && g.gb != nullptr;
+    // gb holds the weight of the norm after the sublayer, or where there is none the other vector to add
+    const float* extra = post ? g.gb : g.x0 ? g.x0 + (size_t)tok * g.ldx : nullptr;
     if constexpr (VEC) {
         const f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
         const float* y = g.y + (size_t)tok * g.ldy;
@@ -86,7 +88,7 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
             if constexpr (PRO == 1) yv[i] = in && have_y ? *reinterpret_cast<const f32x4*>(y + 4 * c) : zero;
             xv[i] = in ? *reinterpret_cast<const f32x4*>(x + 4 * c) : zero;
             if constexpr (PRO == 1) {
-                gb[i] = in && have_y ? *reinterpret_cast<const f32x4*>(g.gb + 4 * c) : zero;
+                gb[i] = in && extra ? *reinterpret_cast<const f32x4*>(extra + 4 * c) : zero;
                 gv[i] = in ? *reinterpret_cast<const f32x4*>(g.g + 4 * c) : zero;
             }
         }
@@ -120,7 +122,7 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     // ---- the vector
     if constexpr (PRO == 1 && VEC) {
         float rs = 0.0f;
-        if (have_y) {
+        if (post) {
             float ss = 0.0f;
 #pragma unroll
             for (int i = 0; i < Q; i++)
@@ -133,7 +135,7 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
         for (int i = 0; i < Q; i++)
 #pragma unroll
             for (int e = 0; e < 4; e++) {
-                if (have_y) xv[i][e] = xv[i][e] + yv[i][e] * rs * gb[i][e];
+                xv[i][e] = post ? xv[i][e] + yv[i][e] * rs * gb[i][e] : xv[i][e] + yv[i][e] + gb[i][e];
                 ss = fma_f(xv[i][e], xv[i][e], ss);
             }
         const float rx = 1.0f / sqrtf(block_sum<4>(ss, nred) / (float)g.k + g.eps);
@@ -155,12 +157,16 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
             const float* y = g.y + (size_t)tok * g.ldy;
             float ss = 0.0f;
             for (int i = t; i < g.k; i += 256) { const float v = y[i]; xs[i] = v; ss = fma_f(v, v, ss); }
-            rs = 1.0f / sqrtf(block_sum<4>(ss, nred) / (float)g.k + g.eps);
+            if (post) rs = 1.0f / sqrtf(block_sum<4>(ss, nred) / (float)g.k + g.eps);
         }
         float ss = 0.0f;
         for (int i = t; i < g.k; i += 256) {
             float v = x[i];
-            if (have_y) v = v + xs[i] * rs * g.gb[i];
+            if (post) v = v + xs[i] * rs * extra[i];
+            else {
+                if (have_y) v += xs[i];
+                if (extra) v += extra[i];
+            }
             xs[i] = v;
             ss = fma_f(v, v, ss);
             if (blockIdx.x == 0 && g.x_new) g.x_new[(size_t)tok * g.ldx + i] = v;
@@ -192,6 +198,11 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
     };
     auto process = [&](int b, int grp) {
         float acc[R];
+        float bias[2] = {0.0f, 0.0f};                     // of the rows that this thread hands out below
+        if (g.bias && t < R) {
+            bias[0] = g.bias[min(grp * R + t, g.n - 1)];
+            bias[1] = g.bias[min(grp * R + t + 1, g.n - 1)];
+        }
 #pragma unroll
         for (int r = 0; r < R; r++) acc[r] = 0.0f;
 #pragma unroll
@@ -212,13 +223,13 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
 #pragma unroll
             for (int i = 0; i < 2; i++) {
                 const int r = min(t + i, R - 1);
-                v[i] = (red[b][r] + red[b][R + r]) + (red[b][2 * R + r] + red[b][3 * R + r]);
+                v[i] = (red[b][r] + red[b][R + r]) + (red[b][2 * R + r] + red[b][3 * R + r]) + bias[i];
             }
             if (row < g.n) {
                 const size_t o = blockIdx.y;
                 if (row >= g.n_split) g.out32[o * g.ldo32 + row - g.n_split] = v[0];
                 else if (!g.glu) g.out[o * g.ldo + row] = v[0];
-                else if ((row & 1) == 0) g.out[o * g.ldo + (row >> 1)] = clamped_glu_f(v[0], v[1], g.limit);
+                else if ((row & 1) == 0) g.out[o * g.ldo + (row >> 1)] = glu_f(g.glu, v[0], v[1], g.limit);
             }
         }
     };

@@ -1,6 +1,9 @@
-// Decoder of floating-point layers (latent attention, gated linear attention, dense or mixture feed-forwards) on one GPU:
-// owns the repacked weights, the slots with the sequences' cached rows and states, and the workspace, and strings the
-// kernels of float_ops.h together.
+// Decoder of floating-point layers (latent attention, attention over shared key/value rows, gated linear attention, dense or
+// mixture feed-forwards) on one GPU: owns the repacked weights, the slots with the sequences' cached rows and states, and
+// the workspace, and strings the kernels of float_ops.h together.
+//
+// A layer run is one pass through a layer: layers inside the loop have several, with the same weights and rows or states of
+// their own.
 //
 // Two schedules over the same weights and slots: up to kSmallTokens tokens go through the one-token linears with float32
 // activations (decode: every quantity that changes between steps is read from the slot's device state, so one captured
@@ -18,14 +21,15 @@ namespace fx {
 constexpr int kSmallTokens = 8;
 constexpr int kPieceTokens = 4096;
 constexpr int kHeadRows = 256;          // rows of logits formed at a time
-constexpr int kAbsorbTokens = 16;       // tokens per launch of the latent-space attention
+constexpr int kAbsorbTokens = 16;       // tokens per launch of the attention kernels for few tokens
 
 static inline int up4(int v) { return (v + 3) / 4 * 4; }
 
 struct HybridLayer {
     flexllm_hybrid_layer d;
-    float *g1 = nullptr, *g1b = nullptr, *g2 = nullptr, *g2b = nullptr;       // 1 + stored weight
-    void *w_in = nullptr, *w_o = nullptr;     // latent: [q; dkv]; gated linear: [q; k; v; g; a1]
+    float *g1 = nullptr, *g1b = nullptr, *g2 = nullptr, *g2b = nullptr;       // effective norm weights
+    void *w_in = nullptr, *w_o = nullptr;     // latent: [q; dkv]; shared key/value: [q; k]; gated linear: [q; k; v; g; a1]
+    float* in_bias = nullptr;                 // [n_in]
     int n_in = 0, n_et = 0, k_o = 0;          // rows of w_in, those that stay in ET, width of w_o's input
     void *uk = nullptr, *uv = nullptr;
     float* latent_norm = nullptr;
@@ -35,13 +39,19 @@ struct HybridLayer {
     void *w_gu = nullptr, *w_d = nullptr;     // dense, or the experts one after the other
     void *w_side = nullptr, *w_sd = nullptr;  // mixture: [shared gate/up; router; shared gate row], shared down
     int n_side = 0;
+    float* kv_norm = nullptr;                 // product of the query and key norms' weights
     LatentDims ld = {};
+    SharedKvDims sd = {};
     GlaDims gd = {};
 };
 
+struct LayerRun { int layer; bool again; };        // again: the embedding output is added ahead of it
+
 struct HybridSlot {
-    std::vector<void*> rows;                  // per layer: cached rows (own or, with kv_from, the other layer's)
-    std::vector<float*> state;                // per layer: gated linear attention state
+    // per layer run
+    std::vector<void*> rows;                  // cached rows (own or, with kv_from, the other layer's)
+    std::vector<float*> inv_rms;              // shared key/value: what the rows' products are multiplied by
+    std::vector<float*> state;                // gated linear attention state
     int* pos = nullptr;                       // device: [0] tokens held, [1] step of the decode loop, [3] error flag
     int length = 0;
 };
@@ -51,6 +61,7 @@ struct HybridSlot {
 struct flexllm_hybrid {
     flexllm_hybrid_config cfg;
     std::vector<fx::HybridLayer> layers;
+    std::vector<fx::LayerRun> runs;
     std::vector<fx::HybridSlot> slots;
     std::vector<void*> owned, pool;           // pool: the many-token workspace
     uint16_t* embed = nullptr;
@@ -58,9 +69,9 @@ struct flexllm_hybrid {
     float* g_final = nullptr;
     // largest sizes over the layers
     int max_et = 0, max_f32 = 0, max_att = 0, max_ff = 0, max_slots_ff = 1, max_shared = 0, max_route = 4, max_experts = 0, max_top = 1;
-    size_t absorbed = 0;                      // scratch floats per token of the latent-space attention
+    size_t absorbed = 0;                      // scratch floats per token of the attention kernels for few tokens
     // one-token workspace
-    float *xa = nullptr, *xb = nullptr, *proj = nullptr, *f32 = nullptr, *att = nullptr, *y = nullptr, *hn = nullptr, *hid = nullptr, *hs = nullptr, *route = nullptr;
+    float *x0 = nullptr, *xa = nullptr, *xb = nullptr, *proj = nullptr, *f32 = nullptr, *att = nullptr, *y = nullptr, *hn = nullptr, *hid = nullptr, *hs = nullptr, *route = nullptr;
     float *pick_w = nullptr, *scratch = nullptr, *logits = nullptr, *hw = nullptr;
     int *pick = nullptr, *want = nullptr;
     float* am_v = nullptr;
@@ -70,7 +81,7 @@ struct flexllm_hybrid {
     int* gen_token = nullptr;
     // many-token workspace
     int rows = 0;
-    float *lx = nullptr, *lf32 = nullptr, *ly = nullptr, *lys = nullptr, *lroute = nullptr, *lgla = nullptr, *lpick_w = nullptr;
+    float *lx0 = nullptr, *lx = nullptr, *lf32 = nullptr, *ly = nullptr, *lys = nullptr, *lroute = nullptr, *lgla = nullptr, *lpick_w = nullptr;
     void *lh = nullptr, *lproj = nullptr, *latt = nullptr, *lhid = nullptr, *lhs = nullptr, *lk = nullptr, *lvt = nullptr, *lhead = nullptr;
     int *lpick = nullptr, *lpos_of = nullptr, *lrow_src = nullptr, *lcounts = nullptr, *lntiles = nullptr;
     int4* ltiles = nullptr;
@@ -127,6 +138,14 @@ struct Packer {
         if (step == 1) next += n;
         return FLEXLLM_OK;
     }
+    // rows of heads that lie `padded` rows apart
+    int put_heads(const uint16_t* src, int heads, int dim, int padded, const char* what) {
+        for (int h = 0; h < heads; h++) {
+            FX_TRY(put(src ? src + (size_t)h * dim * k : nullptr, dim, what));
+            next += padded - dim;
+        }
+        return FLEXLLM_OK;
+    }
     int put_pair(const uint16_t* gate, const uint16_t* up, int n, const char* what) {
         FX_TRY(put(gate, n, what, 2, 0));
         FX_TRY(put(up, n, what, 2, 1));
@@ -134,6 +153,22 @@ struct Packer {
         return FLEXLLM_OK;
     }
 };
+
+static int host_floats(const uint16_t* src, int n, std::vector<float>& out) {
+    std::vector<uint16_t> u(n);
+    FX_HIP(hipMemcpy(u.data(), src, n * sizeof(uint16_t), hipMemcpyDeviceToHost));
+    out.resize(n);
+    for (int i = 0; i < n; i++) {
+        const uint32_t w = (uint32_t)u[i] << 16;
+        memcpy(&out[i], &w, 4);
+    }
+    return FLEXLLM_OK;
+}
+static int own_floats(flexllm_hybrid* m, float*& dst, const std::vector<float>& v) {
+    FX_TRY(own(m, dst, v.size()));
+    FX_HIP(hipMemcpy(dst, v.data(), v.size() * sizeof(float), hipMemcpyHostToDevice));
+    return FLEXLLM_OK;
+}
 
 // Rotation tables: neighbouring pairs; with yarn the frequencies of slow pairs are divided by the factor, with a ramp
 // between the pairs that turn `fast` and `slow` times over the original length, and sine and cosine are scaled.
@@ -178,10 +213,15 @@ static int check_layer(const flexllm_hybrid_config& c, const flexllm_hybrid_laye
             FX_REQUIRE(s.mixer == FLEXLLM_MIX_LATENT && s.kv_from < 0 && s.kv_rank == d.kv_rank && s.rot_dim == d.rot_dim,
                        "hybrid_create: layer %d cannot read the rows of layer %d", i, d.kv_from);
         }
+    } else if (d.mixer == FLEXLLM_MIX_SHARED_KV) {
+        FX_REQUIRE(d.kv_heads > 0 && d.heads % d.kv_heads == 0 && d.vdim == d.dim && d.dim <= 512, "hybrid_create: layer %d: %d heads on %d, dim=%d vdim=%d (at most 512)",
+                   i, d.heads, d.kv_heads, d.dim, d.vdim);
+        FX_REQUIRE(d.temp_coef == 0.0f || d.temp_every > 0, "hybrid_create: layer %d: temp_every=%d", i, d.temp_every);
     } else {
         FX_REQUIRE(d.mixer == FLEXLLM_MIX_GLA && d.a_rank > 0 && d.tau > 0.0f, "hybrid_create: layer %d: mixer=%d a_rank=%d tau=%g", i, d.mixer, d.a_rank, (double)d.tau);
     }
     FX_REQUIRE(d.ff_kind >= FLEXLLM_FF_NONE && d.ff_kind <= FLEXLLM_FF_MOE, "hybrid_create: layer %d: ff_kind=%d", i, d.ff_kind);
+    FX_REQUIRE(d.glu == FLEXLLM_GLU_CLAMPED || d.glu == FLEXLLM_GLU_GELU, "hybrid_create: layer %d: glu=%d", i, d.glu);
     FX_REQUIRE(d.ff_kind == FLEXLLM_FF_NONE || d.ff > 0, "hybrid_create: layer %d: ff=%d", i, d.ff);
     FX_REQUIRE(d.ff_kind != FLEXLLM_FF_MOE || (d.experts > 0 && d.experts <= 1024 && d.top > 0 && d.top <= 32 && d.top <= d.experts && d.shared_ff >= 0),
                "hybrid_create: layer %d: %d experts, top %d", i, d.experts, d.top);
@@ -196,8 +236,8 @@ static int create_layer(flexllm_hybrid* m, int i, const flexllm_hybrid_layer_wei
     const flexllm_hybrid_layer& d = L.d;
     const flexllm_hybrid_config& c = m->cfg;
     const int W = c.width;
-    FX_TRY(own_norm(m, L.g1, w.norm1, W, 1.0f, "norm1"));
-    FX_TRY(own_norm(m, L.g1b, w.norm1b, W, 1.0f, "norm1b"));
+    FX_TRY(own_norm(m, L.g1, w.norm1, W, c.norm_add, "norm1"));
+    if (c.post_norms) FX_TRY(own_norm(m, L.g1b, w.norm1b, W, c.norm_add, "norm1b"));
     Packer<ET> in(m, W), out(m, d.heads * d.vdim);
     if (d.mixer == FLEXLLM_MIX_LATENT) {
         const int nq = d.heads * (d.dim + d.rot_dim), nk = d.kv_from < 0 ? d.kv_rank + d.rot_dim : 0;
@@ -227,6 +267,37 @@ static int create_layer(flexllm_hybrid* m, int i, const flexllm_hybrid_layer_wei
         if (!L.cos_t) FX_TRY(rotation_tables(m, d, L.cos_t, L.sin_t));
         const size_t a = latent_absorbed_scratch(ld);
         if (a > m->absorbed) m->absorbed = a;
+    } else if (d.mixer == FLEXLLM_MIX_SHARED_KV) {
+        SharedKvDims& s = L.sd;
+        s.heads = d.heads; s.kv_heads = d.kv_heads; s.dim = d.dim; s.dimp = pad8(d.dim); s.sink = d.sink; s.scale = d.scale;
+        s.temp_coef = d.temp_coef; s.temp_every = d.temp_every; s.eps = c.eps; s.capacity = c.max_pos;
+        L.n_et = d.heads * s.dimp;
+        L.n_in = L.n_et + d.kv_heads * s.dimp;
+        FX_TRY(in.alloc(L.n_in));
+        FX_TRY(in.put_heads(w.q, d.heads, d.dim, s.dimp, "mix.q"));
+        FX_TRY(in.put_heads(w.k, d.kv_heads, d.dim, s.dimp, "mix.k"));
+        std::vector<float> v, u;
+        if (w.q_bias || w.k_bias) {
+            std::vector<float> bias(L.n_in, 0.0f);
+            auto spread = [&](const uint16_t* src, int heads, int at) {
+                if (!src) return FLEXLLM_OK;
+                FX_TRY(host_floats(src, heads * d.dim, v));
+                for (int h = 0; h < heads; h++)
+                    for (int e = 0; e < d.dim; e++) bias[at + h * s.dimp + e] = v[h * d.dim + e];
+                return FLEXLLM_OK;
+            };
+            FX_TRY(spread(w.q_bias, d.heads, 0));
+            FX_TRY(spread(w.k_bias, d.kv_heads, L.n_et));
+            FX_TRY(own_floats(m, L.in_bias, bias));
+        }
+        FX_REQUIRE(w.q_norm && w.k_norm, "hybrid_create: missing tensor mix.q.norm or mix.k.norm");
+        FX_TRY(host_floats(w.q_norm, d.dim, v));
+        FX_TRY(host_floats(w.k_norm, d.dim, u));
+        for (int e = 0; e < d.dim; e++) v[e] *= u[e];
+        v.resize(s.dimp, 0.0f);
+        FX_TRY(own_floats(m, L.kv_norm, v));
+        const size_t a = shared_kv_scratch(s);
+        if (a > m->absorbed) m->absorbed = a;
     } else {
         const int HD = d.heads * d.dim, HV = d.heads * d.vdim;
         L.n_et = 2 * HD + 2 * HV;
@@ -252,12 +323,12 @@ static int create_layer(flexllm_hybrid* m, int i, const flexllm_hybrid_layer_wei
     FX_TRY(out.put(w.o, W, "mix.o"));
     L.w_o = out.dst;
     auto grow = [](int& v, int n) { if (n > v) v = n; };
-    grow(m->max_et, L.n_et);
+    grow(m->max_et, up4(L.n_et));
     grow(m->max_f32, L.n_in - L.n_et);
     grow(m->max_att, L.k_o);
     if (d.ff_kind == FLEXLLM_FF_NONE) return FLEXLLM_OK;
-    FX_TRY(own_norm(m, L.g2, w.norm2, W, 1.0f, "norm2"));
-    FX_TRY(own_norm(m, L.g2b, w.norm2b, W, 1.0f, "norm2b"));
+    FX_TRY(own_norm(m, L.g2, w.norm2, W, c.norm_add, "norm2"));
+    if (c.post_norms) FX_TRY(own_norm(m, L.g2b, w.norm2b, W, c.norm_add, "norm2b"));
     Packer<ET> gu(m, W), dn(m, d.ff);
     const int E = d.ff_kind == FLEXLLM_FF_MOE ? d.experts : 1;
     FX_TRY(gu.alloc((size_t)E * 2 * d.ff));
@@ -302,24 +373,40 @@ static int create_model(flexllm_hybrid* m, const flexllm_hybrid_weights& w, cons
     FX_REQUIRE(w.embed && w.head && w.final_norm, "hybrid_create: missing tensor embed, head or final.norm");
     FX_TRY(own(m, m->embed, (size_t)c.vocab * W));
     FX_HIP(hipMemcpy(m->embed, w.embed, (size_t)c.vocab * W * 2, hipMemcpyDeviceToDevice));
-    FX_TRY(own_norm(m, m->g_final, w.final_norm, W, 1.0f, "final.norm"));
-    Packer<ET> head(m, W);
-    FX_TRY(head.alloc(c.vocab));
-    FX_TRY(head.put(w.head, c.vocab, "head"));
-    m->head = head.dst;
+    FX_TRY(own_norm(m, m->g_final, w.final_norm, W, c.norm_add, "final.norm"));
+    if (w.head == w.embed && std::is_same<ET, bf16_t>::value && pad_k(W) == W) {
+        m->head = m->embed;                               // tied, and already in the head's layout
+    } else {
+        Packer<ET> head(m, W);
+        FX_TRY(head.alloc(c.vocab));
+        FX_TRY(head.put(w.head, c.vocab, "head"));
+        m->head = head.dst;
+    }
     for (int i = 0; i < c.layers; i++) FX_TRY(create_layer<ET>(m, i, lw[i]));
     m->slots.resize(c.slots);
     for (HybridSlot& s : m->slots) {
-        s.rows.resize(c.layers); s.state.resize(c.layers);
+        const int n = (int)m->runs.size();
+        s.rows.resize(n); s.inv_rms.resize(n); s.state.resize(n);
         FX_TRY(own(m, s.pos, 8));
-        for (int i = 0; i < c.layers; i++) {
+        std::vector<int> latest(c.layers, -1);            // the last run of a layer so far
+        for (int r = 0; r < n; r++) {
+            const int i = m->runs[r].layer;
             const HybridLayer& L = m->layers[i];
-            if (L.d.mixer == FLEXLLM_MIX_GLA) FX_TRY(own(m, s.state[i], (size_t)L.d.heads * L.d.dim * L.d.vdim));
-            else if (L.d.kv_from >= 0) s.rows[i] = s.rows[L.d.kv_from];
-            else FX_TRY(halloc(m->owned, &s.rows[i], (size_t)c.max_pos * L.ld.ldc * sizeof(ET)));
+            if (L.d.mixer == FLEXLLM_MIX_GLA) {
+                FX_TRY(own(m, s.state[r], (size_t)L.d.heads * L.d.dim * L.d.vdim));
+            } else if (L.d.mixer == FLEXLLM_MIX_SHARED_KV) {
+                FX_TRY(halloc(m->owned, &s.rows[r], (size_t)L.sd.kv_heads * c.max_pos * L.sd.dimp * sizeof(ET)));
+                FX_TRY(own(m, s.inv_rms[r], (size_t)L.sd.kv_heads * c.max_pos));
+            } else if (L.d.kv_from >= 0) {
+                s.rows[r] = s.rows[latest[L.d.kv_from]];
+            } else {
+                FX_TRY(halloc(m->owned, &s.rows[r], (size_t)c.max_pos * L.ld.ldc * sizeof(ET)));
+            }
+            latest[i] = r;
         }
     }
     const size_t T = kSmallTokens;
+    FX_TRY(own(m, m->x0, T * W));
     FX_TRY(own(m, m->xa, T * W));
     FX_TRY(own(m, m->xb, T * W));
     FX_TRY(own(m, m->hn, T * W));
@@ -365,7 +452,7 @@ static int many_workspace(flexllm_hybrid* m, int rows) {
             kv = (kv + 127) / 64 * 64;
             if (kv * L.d.heads * L.d.dim > k_el) k_el = kv * L.d.heads * L.d.dim;
             if (kv * L.d.heads * L.d.vdim > vt_el) vt_el = kv * L.d.heads * L.d.vdim;
-        } else if (gla_chunks_ok(L.gd)) {
+        } else if (L.d.mixer == FLEXLLM_MIX_GLA && gla_chunks_ok(L.gd)) {
             const size_t g = gla_chunk_scratch(L.gd, (int)R);
             if (g > gla) gla = g;
         }
@@ -374,6 +461,7 @@ static int many_workspace(flexllm_hybrid* m, int rows) {
     auto pool_et = [&](void*& p, size_t count) { return halloc(m->pool, &p, count * sizeof(ET)); };
     const size_t top = m->max_experts ? m->max_top : 1;
     FX_TRY(pool(m->lx, R * W));
+    if (c.loop_times > 1) FX_TRY(pool(m->lx0, R * W));
     FX_TRY(pool(m->lf32, R * (m->max_f32 + 4)));
     FX_TRY(pool(m->ly, R * W));
     FX_TRY(pool_et(m->lh, R * pad_k((int)W)));
@@ -401,26 +489,44 @@ static int many_workspace(flexllm_hybrid* m, int rows) {
 }
 
 // ---- one to kSmallTokens tokens --------------------------------------------------------------------------------------
-struct Pending { const float* gb = nullptr; };            // the last sublayer's output in y still has to be added
+struct Pending { bool on = false; const float* gb = nullptr; };      // the last sublayer's output in y still has to be added
 
 template <typename ET>
 static int run_small(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, const int* want, int n_want, float* logits, float* layers_out, hipStream_t st) {
     const flexllm_hybrid_config& c = m->cfg;
     const int W = c.width, kw = pad_k(W);
-    float *x = m->xa, *other = m->xb;
+    float *x = m->x0, *other = m->xa;                     // the embedding output stays in x0, later residuals alternate
     Pending pend;
-    FX_TRY(embed_rows_bf16(as_bf16(m->embed), tokens, T, x, W, c.vocab, &s.pos[3], st));
+    FX_TRY(embed_rows_bf16(as_bf16(m->embed), c.embed_scale, tokens, T, x, W, c.vocab, &s.pos[3], st));
+    auto moved = [&] {                                    // the residual now is where `other` was
+        x = other;
+        other = x == m->xa ? m->xb : m->xa;
+        pend = Pending();
+    };
+    auto settle = [&] {                                   // take the pending output in, without a norm behind it
+        if (!pend.on) return FLEXLLM_OK;
+        RowArgs r;
+        r.x = x; r.x_new = other; r.y = m->y; r.ldy = W; r.gb = pend.gb; r.eps = c.eps; r.width = W; r.rows = T;
+        const int rc = norm_rows<ET>(r, st);
+        moved();
+        return rc;
+    };
+    auto pending = [&](const float* gb) { pend.on = true; pend.gb = gb; };
     auto base = [&](const void* w, int n, int k) {
         GemvArgs a;
         a.w = w; a.n = n; a.k = k; a.kpad = pad_k(k); a.eps = c.eps;
         return a;
     };
-    // linear on norm(x + pending)
-    auto norm_linear = [&](GemvArgs a, const float* g) {
+    // linear on norm(x + pending [+ x0])
+    auto norm_linear = [&](GemvArgs a, const float* g, bool add_x0 = false) {
+        if (add_x0 && pend.gb) FX_TRY(settle());          // the kernel takes a norm's weight or x0
         a.x = x; a.ldx = W; a.g = g;
-        if (pend.gb) { a.y = m->y; a.ldy = W; a.gb = pend.gb; a.x_new = other; }
+        if (pend.on) { a.y = m->y; a.ldy = W; a.gb = pend.gb; }
+        if (add_x0) a.x0 = m->x0;
+        const bool changes = pend.on || add_x0;
+        if (changes) a.x_new = other;
         const int rc = gemv_float<ET>(a, 1, T, st);
-        if (pend.gb) { float* t = x; x = other; other = t; pend.gb = nullptr; }
+        if (changes) moved();
         return rc;
     };
     auto plain_linear = [&](const void* w, int n, int k, const float* v, int ldv, float* out) {
@@ -428,37 +534,44 @@ static int run_small(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T,
         a.x = v; a.ldx = ldv; a.n_split = 0; a.out32 = out; a.ldo32 = n;
         return gemv_float<ET>(a, 0, T, st);
     };
-    for (int i = 0; i < c.layers; i++) {
-        const HybridLayer& L = m->layers[i];
+    const int runs = (int)m->runs.size();
+    for (int r = 0; r < runs; r++) {
+        const HybridLayer& L = m->layers[m->runs[r].layer];
         const int nf = L.n_in - L.n_et;
+        if (layers_out && r > 0) {
+            FX_TRY(settle());
+            FX_HIP(hipMemcpyAsync(layers_out + (size_t)(r - 1) * T * W, x, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
+        }
         GemvArgs a = base(L.w_in, L.n_in, W);
-        a.n_split = L.n_et; a.out = m->proj; a.ldo = m->max_et; a.out32 = m->f32; a.ldo32 = nf;
-        FX_TRY(norm_linear(a, L.g1));
-        if (layers_out && i > 0) FX_HIP(hipMemcpyAsync(layers_out + (size_t)(i - 1) * T * W, x, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
-        if (L.d.mixer == FLEXLLM_MIX_LATENT) {
-            ET* rows = static_cast<ET*>(s.rows[i]);
+        a.n_split = L.n_et; a.out = m->proj; a.ldo = m->max_et; a.out32 = m->f32; a.ldo32 = nf; a.bias = L.in_bias;
+        FX_TRY(norm_linear(a, L.g1, m->runs[r].again));
+        if (L.d.mixer == FLEXLLM_MIX_SHARED_KV) {
+            const SharedKvRows<ET> rows = {static_cast<ET*>(s.rows[r]), s.inv_rms[r]};
+            FX_TRY(shared_kv_splits<ET>(L.sd, m->proj, m->max_et, m->f32, nf, L.kv_norm, rows, s.pos, 0, T, m->scratch, m->att, m->max_att, 1, st));
+        } else if (L.d.mixer == FLEXLLM_MIX_LATENT) {
+            ET* rows = static_cast<ET*>(s.rows[r]);
             FX_TRY(latent_decode<ET>(L.ld, m->proj, m->max_et, nf ? m->f32 : nullptr, nf, L.latent_norm, L.cos_t, L.sin_t, static_cast<ET*>(L.uk),
                                      static_cast<ET*>(L.uv), rows, s.pos, T, m->scratch, m->att, m->max_att, st));
         } else {
-            FX_TRY(gla_steps<ET>(L.gd, m->proj, m->max_et, 1, m->f32, nf, static_cast<ET*>(L.a2), L.a2_bias, L.head_norm, s.state[i], s.pos, 0, T, m->att, m->max_att, 1, st));
+            FX_TRY(gla_steps<ET>(L.gd, m->proj, m->max_et, 1, m->f32, nf, static_cast<ET*>(L.a2), L.a2_bias, L.head_norm, s.state[r], s.pos, 0, T, m->att, m->max_att, 1, st));
         }
         FX_TRY(plain_linear(L.w_o, W, L.k_o, m->att, m->max_att, m->y));
-        pend.gb = L.g1b;
+        pending(L.g1b);
         if (L.d.ff_kind == FLEXLLM_FF_DENSE) {
             a = base(L.w_gu, 2 * L.d.ff, W);
-            a.n_split = 2 * L.d.ff; a.glu = 1; a.limit = L.d.limit; a.out = m->hid; a.ldo = L.d.ff;
+            a.n_split = 2 * L.d.ff; a.glu = 1 + L.d.glu; a.limit = L.d.limit; a.out = m->hid; a.ldo = L.d.ff;
             FX_TRY(norm_linear(a, L.g2));
             FX_TRY(plain_linear(L.w_d, W, L.d.ff, m->hid, L.d.ff, m->y));
-            pend.gb = L.g2b;
+            pending(L.g2b);
         } else if (L.d.ff_kind == FLEXLLM_FF_MOE) {
             const int sf = L.d.shared_ff, ldr = L.n_side - 2 * sf;
             a = base(L.w_side, L.n_side, W);
-            a.n_split = 2 * sf; a.glu = 1; a.limit = L.d.shared_limit; a.out = m->hs; a.ldo = sf; a.out32 = m->route; a.ldo32 = ldr;
+            a.n_split = 2 * sf; a.glu = 1 + L.d.glu; a.limit = L.d.shared_limit; a.out = m->hs; a.ldo = sf; a.out32 = m->route; a.ldo32 = ldr;
             a.h_out = m->hn; a.ldh = W;
             FX_TRY(norm_linear(a, L.g2));
             a = base(L.w_gu, 2 * L.d.ff, W);
             a.w_stride = (size_t)2 * L.d.ff * kw;
-            a.n_split = 2 * L.d.ff; a.glu = 1; a.limit = L.d.limit; a.out = m->hid; a.ldo = L.d.ff; a.x = m->hn; a.ldx = W;
+            a.n_split = 2 * L.d.ff; a.glu = 1 + L.d.glu; a.limit = L.d.limit; a.out = m->hid; a.ldo = L.d.ff; a.x = m->hn; a.ldx = W;
             a.route = m->route; a.ld_route = ldr; a.experts = L.d.experts; a.top = L.d.top; a.pick = m->pick; a.pick_w = m->pick_w;
             FX_TRY(gemv_float<ET>(a, 2, T, st));
             MoeDownArgs b;
@@ -467,7 +580,7 @@ static int run_small(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T,
             b.route = m->route; b.ld_route = ldr; b.experts = L.d.experts; b.top = L.d.top; b.pick = m->pick; b.pick_w = m->pick_w;
             b.y = m->y; b.ldy = W; b.n = W;
             FX_TRY(moe_down_small<ET>(b, T, st));
-            pend.gb = L.g2b;
+            pending(L.g2b);
         }
     }
     if (n_want == 1 && T == 1 && !layers_out) {
@@ -476,10 +589,8 @@ static int run_small(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T,
         return norm_linear(a, m->g_final);
     }
     if (!n_want && !layers_out) return FLEXLLM_OK;
-    RowArgs r;
-    r.x = x; r.y = m->y; r.ldy = W; r.gb = pend.gb; r.eps = c.eps; r.width = W; r.rows = T;
-    FX_TRY(norm_rows<ET>(r, st));
-    if (layers_out) FX_HIP(hipMemcpyAsync(layers_out + (size_t)(c.layers - 1) * T * W, x, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
+    FX_TRY(settle());
+    if (layers_out) FX_HIP(hipMemcpyAsync(layers_out + (size_t)(runs - 1) * T * W, x, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
     if (!n_want) return FLEXLLM_OK;
     FX_HIP(hipMemcpyAsync(m->want, want, sizeof(int) * n_want, hipMemcpyHostToDevice, st));
     RowArgs f;
@@ -497,11 +608,13 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
     const flexllm_hybrid_config& c = m->cfg;
     const int W = c.width, kw = pad_k(W), ldp = (m->max_et + 7) / 8 * 8, pos0 = s.length;
     FX_TRY(many_workspace<ET>(m, T));
-    FX_TRY(embed_rows_bf16(as_bf16(m->embed), tokens, T, m->lx, W, c.vocab, &s.pos[3], st));
+    float* x = m->lx0 ? m->lx0 : m->lx;                   // with a loop, the embedding output stays in lx0
+    FX_TRY(embed_rows_bf16(as_bf16(m->embed), c.embed_scale, tokens, T, x, W, c.vocab, &s.pos[3], st));
     RowArgs pend;                                         // what the next row kernel has to take in first
     auto rows_h = [&](const float* g) {
         RowArgs r = pend;
-        r.x = m->lx; r.eps = c.eps; r.width = W; r.rows = T;
+        r.x = x; r.eps = c.eps; r.width = W; r.rows = T;
+        if (r.y || r.ys || r.x0) r.x_new = x = m->lx;
         if (g) { r.h = m->lh; r.ldh = kw; r.g = g; }
         pend = RowArgs();
         return norm_rows<ET>(r, st);
@@ -516,17 +629,35 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
         g.n_split = 0; g.y32 = m->ly; g.ldy32 = W;
         return gemm_float<ET>(g, st);
     };
-    for (int i = 0; i < c.layers; i++) {
-        const HybridLayer& L = m->layers[i];
+    const int runs = (int)m->runs.size();
+    for (int r = 0; r < runs; r++) {
+        const HybridLayer& L = m->layers[m->runs[r].layer];
         const int nf = L.n_in - L.n_et, lda = pad_k(L.k_o);
+        if (layers_out && r > 0) {
+            FX_TRY(rows_h(nullptr));
+            FX_HIP(hipMemcpyAsync(layers_out + (size_t)(r - 1) * layer_stride, x, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
+        }
+        if (m->runs[r].again) pend.x0 = m->lx0;
         FX_TRY(rows_h(L.g1));
-        if (layers_out && i > 0) FX_HIP(hipMemcpyAsync(layers_out + (size_t)(i - 1) * layer_stride, m->lx, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
         GemmArgs g = gemm(m->lh, kw, L.w_in, T, L.n_in, W);
-        g.n_split = L.n_et; g.y = m->lproj; g.ldy = ldp; g.y32 = m->lf32; g.ldy32 = nf;
+        g.n_split = L.n_et; g.y = m->lproj; g.ldy = ldp; g.y32 = m->lf32; g.ldy32 = nf; g.bias = L.in_bias;
         FX_TRY(gemm_float<ET>(g, st));
         ET *proj = static_cast<ET*>(m->lproj), *att = static_cast<ET*>(m->latt);
-        if (L.d.mixer == FLEXLLM_MIX_LATENT) {
-            ET *cache = static_cast<ET*>(s.rows[i]), *uk = static_cast<ET*>(L.uk), *uv = static_cast<ET*>(L.uv);
+        if (L.d.mixer == FLEXLLM_MIX_SHARED_KV) {
+            const SharedKvRows<ET> rows = {static_cast<ET*>(s.rows[r]), s.inv_rms[r]};
+            FX_TRY(shared_kv_store<ET>(L.sd, m->lf32, nf, rows, s.pos, T, st));
+            bool flash = false;
+            if constexpr (std::is_same<ET, bf16_t>::value) {
+                flash = shared_kv_flash_ok(L.sd);
+                if (flash) FX_TRY(shared_kv_flash(L.sd, proj, ldp, L.kv_norm, rows, pos0, T, att, lda, st));
+            }
+            if (!flash)
+                for (int t0 = 0; t0 < T; t0 += kAbsorbTokens) {
+                    const int n = T - t0 < kAbsorbTokens ? T - t0 : kAbsorbTokens;
+                    FX_TRY(shared_kv_splits<ET>(L.sd, proj + (size_t)t0 * ldp, ldp, nullptr, 0, L.kv_norm, rows, s.pos, t0, n, m->scratch, att + (size_t)t0 * lda, lda, 0, st));
+                }
+        } else if (L.d.mixer == FLEXLLM_MIX_LATENT) {
+            ET *cache = static_cast<ET*>(s.rows[r]), *uk = static_cast<ET*>(L.uk), *uv = static_cast<ET*>(L.uv);
             FX_TRY(latent_store<ET>(L.ld, proj, ldp, nf ? m->lf32 : nullptr, nf, L.latent_norm, L.cos_t, L.sin_t, cache, s.pos, T, st));
             bool flash = false;
             if constexpr (std::is_same<ET, bf16_t>::value) {
@@ -551,9 +682,9 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
                     FX_TRY(latent_absorbed<ET>(L.ld, proj + (size_t)t0 * ldp, ldp, uk, uv, cache, s.pos, t0, n, m->scratch, att + (size_t)t0 * lda, lda, st));
                 }
         } else if (gla_chunks_ok(L.gd)) {
-            FX_TRY(gla_chunks<ET>(L.gd, proj, ldp, m->lf32, nf, static_cast<ET*>(L.a2), L.a2_bias, L.head_norm, s.state[i], s.pos, T, m->lgla, att, lda, st));
+            FX_TRY(gla_chunks<ET>(L.gd, proj, ldp, m->lf32, nf, static_cast<ET*>(L.a2), L.a2_bias, L.head_norm, s.state[r], s.pos, T, m->lgla, att, lda, st));
         } else {
-            FX_TRY(gla_steps<ET>(L.gd, proj, ldp, 0, m->lf32, nf, static_cast<ET*>(L.a2), L.a2_bias, L.head_norm, s.state[i], s.pos, 0, T, att, lda, 0, st));
+            FX_TRY(gla_steps<ET>(L.gd, proj, ldp, 0, m->lf32, nf, static_cast<ET*>(L.a2), L.a2_bias, L.head_norm, s.state[r], s.pos, 0, T, att, lda, 0, st));
         }
         FX_TRY(to_y(att, lda, L.w_o, L.k_o));
         pend.y = m->ly; pend.ldy = W; pend.gb = L.g1b;
@@ -562,7 +693,7 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
         FX_TRY(rows_h(L.g2));
         if (L.d.ff_kind == FLEXLLM_FF_DENSE) {
             g = gemm(m->lh, kw, L.w_gu, T, 2 * L.d.ff, W);
-            g.n_split = 2 * L.d.ff; g.glu = 1; g.limit = L.d.limit; g.y = m->lhid; g.ldy = kf;
+            g.n_split = 2 * L.d.ff; g.glu = 1 + L.d.glu; g.limit = L.d.limit; g.y = m->lhid; g.ldy = kf;
             FX_TRY(gemm_float<ET>(g, st));
             FX_TRY(to_y(m->lhid, kf, L.w_d, L.d.ff));
             pend.y = m->ly; pend.ldy = W; pend.gb = L.g2b;
@@ -570,7 +701,7 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
         }
         const int sf = L.d.shared_ff, ldr = L.n_side - 2 * sf, top = L.d.top, ks = pad_k(sf > 0 ? sf : 1);
         g = gemm(m->lh, kw, L.w_side, T, L.n_side, W);
-        g.n_split = 2 * sf; g.glu = 1; g.limit = L.d.shared_limit; g.y = m->lhs; g.ldy = ks; g.y32 = m->lroute; g.ldy32 = ldr;
+        g.n_split = 2 * sf; g.glu = 1 + L.d.glu; g.limit = L.d.shared_limit; g.y = m->lhs; g.ldy = ks; g.y32 = m->lroute; g.ldy32 = ldr;
         FX_TRY(gemm_float<ET>(g, st));
         const int tile = gemm_group_tile_rows(T * top / L.d.experts);
         MoePlan p;
@@ -580,7 +711,7 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
         int max_tiles = T * top / tile + L.d.experts;
         if (max_tiles > T * top) max_tiles = T * top;
         g = gemm(m->lh, kw, L.w_gu, T * top, 2 * L.d.ff, W);
-        g.n_split = 2 * L.d.ff; g.glu = 1; g.limit = L.d.limit; g.y = m->lhid; g.ldy = kf;
+        g.n_split = 2 * L.d.ff; g.glu = 1 + L.d.glu; g.limit = L.d.limit; g.y = m->lhid; g.ldy = kf;
         g.row_src = m->lrow_src; g.tiles = m->ltiles; g.n_tiles = m->lntiles; g.max_tiles = max_tiles; g.w_stride = (size_t)2 * L.d.ff * kw;
         FX_TRY(gemm_grouped<ET>(g, tile, st));
         g = gemm(m->lhid, kf, L.w_d, T * top, W, L.d.ff);
@@ -595,13 +726,13 @@ static int run_many(flexllm_hybrid* m, HybridSlot& s, const int* tokens, int T, 
     }
     if (!n_want && !layers_out) return FLEXLLM_OK;
     FX_TRY(rows_h(nullptr));
-    if (layers_out) FX_HIP(hipMemcpyAsync(layers_out + (size_t)(c.layers - 1) * layer_stride, m->lx, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
+    if (layers_out) FX_HIP(hipMemcpyAsync(layers_out + (size_t)(runs - 1) * layer_stride, x, sizeof(float) * T * W, hipMemcpyDeviceToDevice, st));
     if (!n_want) return FLEXLLM_OK;
     FX_HIP(hipMemcpyAsync(m->want, want, sizeof(int) * n_want, hipMemcpyHostToDevice, st));
     for (int r0 = 0; r0 < n_want; r0 += kHeadRows) {
         const int n = n_want - r0 < kHeadRows ? n_want - r0 : kHeadRows;
         RowArgs f;
-        f.x = m->lx; f.eps = c.eps; f.width = W; f.rows = n; f.rows_src = m->want + r0; f.g = m->g_final;
+        f.x = x; f.eps = c.eps; f.width = W; f.rows = n; f.rows_src = m->want + r0; f.g = m->g_final;
         if (n_want <= kSmallTokens) {
             f.h = m->hw; f.ldh = W; f.h_f32 = 1;
             FX_TRY(norm_rows<ET>(f, st));
@@ -677,11 +808,18 @@ int flexllm_hybrid_create(flexllm_hybrid** out, const flexllm_hybrid_config* cfg
     FX_REQUIRE(out && cfg && layers && w && lw, "hybrid_create: null pointer");
     FX_REQUIRE(cfg->layers > 0 && cfg->width > 0 && cfg->width <= 15360 && cfg->vocab > 0 && cfg->max_pos > 0 && cfg->slots > 0 && (cfg->dtype == 0 || cfg->dtype == 1),
                "hybrid_create: layers=%d width=%d vocab=%d max_pos=%d slots=%d dtype=%d", cfg->layers, cfg->width, cfg->vocab, cfg->max_pos, cfg->slots, cfg->dtype);
+    FX_REQUIRE(cfg->loop_times == 1 || (cfg->loop_times > 1 && cfg->loop_start >= 0 && cfg->loop_start <= cfg->loop_stop && cfg->loop_stop <= cfg->layers),
+               "hybrid_create: layers %d .. %d run %d times", cfg->loop_start, cfg->loop_stop, cfg->loop_times);
     for (int i = 0; i < cfg->layers; i++) FX_TRY(check_layer(*cfg, layers, i));
     flexllm_hybrid* m = new flexllm_hybrid();
     m->cfg = *cfg;
     m->layers.resize(cfg->layers);
+    const int start = cfg->loop_times > 1 ? cfg->loop_start : 0, stop = cfg->loop_times > 1 ? cfg->loop_stop : 0;
     for (int i = 0; i < cfg->layers; i++) m->layers[i].d = layers[i];
+    for (int i = 0; i < start; i++) m->runs.push_back({i, false});
+    for (int k = 0; k < cfg->loop_times; k++)
+        for (int i = start; i < stop; i++) m->runs.push_back({i, k > 0 && i == start});
+    for (int i = stop; i < cfg->layers; i++) m->runs.push_back({i, false});
     const int rc = cfg->dtype == 0 ? create_model<bf16_t>(m, *w, lw) : create_model<float>(m, *w, lw);
     if (rc) { flexllm_hybrid_destroy(m); return rc; }
     *out = m;

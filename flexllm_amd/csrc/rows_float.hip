@@ -32,7 +32,7 @@ int widen_rows(const bf16_t* src, float* dst, int n, float add, hipStream_t st) 
 }
 
 // Ids outside [0, vocab) are replaced by 0 and reported through *err = 2, as in embed_rows_kernel.
-static __global__ __launch_bounds__(256) void embed_bf16_kernel(const bf16_t* __restrict__ table, const int* __restrict__ tokens, float* __restrict__ x,
+static __global__ __launch_bounds__(256) void embed_bf16_kernel(const bf16_t* __restrict__ table, float scale, const int* __restrict__ tokens, float* __restrict__ x,
                                                                 int width, int vocab, int* __restrict__ err) {
     int tk = tokens[blockIdx.x];
     if ((unsigned)tk >= (unsigned)vocab) {
@@ -40,10 +40,10 @@ static __global__ __launch_bounds__(256) void embed_bf16_kernel(const bf16_t* __
         tk = 0;
     }
     const bf16_t* s = table + (size_t)tk * width;
-    for (int i = threadIdx.x; i < width; i += 256) x[(size_t)blockIdx.x * width + i] = (float)s[i];
+    for (int i = threadIdx.x; i < width; i += 256) x[(size_t)blockIdx.x * width + i] = (float)s[i] * scale;
 }
-int embed_rows_bf16(const bf16_t* table, const int* tokens, int n, float* x, int width, int vocab, int* err, hipStream_t st) {
-    embed_bf16_kernel<<<n, 256, 0, st>>>(table, tokens, x, width, vocab, err);
+int embed_rows_bf16(const bf16_t* table, float scale, const int* tokens, int n, float* x, int width, int vocab, int* err, hipStream_t st) {
+    embed_bf16_kernel<<<n, 256, 0, st>>>(table, scale, tokens, x, width, vocab, err);
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
 }
@@ -67,9 +67,10 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(RowArgs a) {
     extern __shared__ float row[];
     __shared__ float red[4];
     const int t = threadIdx.x, r = blockIdx.x;
-    float* x = a.x + (size_t)(a.rows_src ? a.rows_src[r] : r) * a.width;
+    const float* x = a.x + (size_t)(a.rows_src ? a.rows_src[r] : r) * a.width;
+    float* x_new = (a.x_new ? a.x_new : a.x) + (size_t)r * a.width;
     const bool mix = a.ys != nullptr, have_y = a.y || mix;
-    if (have_y) {
+    if (have_y || a.x0) {
         float sg = 1.0f;
         if (mix && a.y) sg = sigmoid_f(a.route[(size_t)r * a.ld_route + a.experts]);
         float ss = 0.0f;
@@ -78,17 +79,19 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(RowArgs a) {
             if (mix) {
                 for (int k = 0; k < a.top; k++) v = fma_f(a.pick_w[r * a.top + k], a.ys[(size_t)a.pos_of[r * a.top + k] * a.ldy + i], v);
                 if (a.y) v = fma_f(sg, a.y[(size_t)r * a.ldy + i], v);
-            } else {
+            } else if (a.y) {
                 v = a.y[(size_t)r * a.ldy + i];
             }
             row[i] = v;
             ss = fma_f(v, v, ss);
         }
-        const float rs = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)a.width + a.eps);
+        const bool post = have_y && a.gb;
+        const float rs = post ? 1.0f / sqrtf(block_sum<4>(ss, red) / (float)a.width + a.eps) : 1.0f;
         for (int i = t; i < a.width; i += 256) {
-            const float v = x[i] + row[i] * rs * a.gb[i];
+            float v = x[i] + (post ? row[i] * rs * a.gb[i] : row[i]);
+            if (a.x0) v += a.x0[(size_t)r * a.width + i];
             row[i] = v;
-            if (!a.rows_src) x[i] = v;
+            if (!a.rows_src) x_new[i] = v;
         }
     } else {
         for (int i = t; i < a.width; i += 256) row[i] = x[i];
@@ -111,7 +114,8 @@ template <typename ET, int V>
 __global__ __launch_bounds__(256) void norm_rows_vec_kernel(RowArgs a) {
     __shared__ float red[4];
     const int t = threadIdx.x, r = blockIdx.x, n4 = a.width >> 2;
-    float* x = a.x + (size_t)(a.rows_src ? a.rows_src[r] : r) * a.width;
+    const float* x = a.x + (size_t)(a.rows_src ? a.rows_src[r] : r) * a.width;
+    float* x_new = (a.x_new ? a.x_new : a.x) + (size_t)r * a.width;
     const bool mix = a.ys != nullptr, have_y = a.y || mix;
     f32x4 v[V];
 #pragma unroll
@@ -119,7 +123,7 @@ __global__ __launch_bounds__(256) void norm_rows_vec_kernel(RowArgs a) {
         const int c = t + i * 256;
         v[i] = c < n4 ? *reinterpret_cast<const f32x4*>(x + c * 4) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
     }
-    if (have_y) {
+    if (have_y || a.x0) {
         f32x4 y[V];
         float ss = 0.0f, sg = 1.0f;
         if (mix && a.y) sg = sigmoid_f(a.route[(size_t)r * a.ld_route + a.experts]);
@@ -140,22 +144,33 @@ __global__ __launch_bounds__(256) void norm_rows_vec_kernel(RowArgs a) {
 #pragma unroll
                         for (int e = 0; e < 4; e++) y[i][e] = fma_f(sg, u[e], y[i][e]);
                     }
-                } else {
+                } else if (a.y) {
                     y[i] = *reinterpret_cast<const f32x4*>(a.y + (size_t)r * a.ldy + c * 4);
                 }
             }
 #pragma unroll
             for (int e = 0; e < 4; e++) ss = fma_f(y[i][e], y[i][e], ss);
         }
-        const float rs = 1.0f / sqrtf(block_sum<4>(ss, red) / (float)a.width + a.eps);
+        const bool post = have_y && a.gb;
+        const float rs = post ? 1.0f / sqrtf(block_sum<4>(ss, red) / (float)a.width + a.eps) : 1.0f;
 #pragma unroll
         for (int i = 0; i < V; i++) {
             const int c = t + i * 256;
             if (c >= n4) continue;
-            const f32x4 gb = *reinterpret_cast<const f32x4*>(a.gb + c * 4);
+            if (post) {
+                const f32x4 gb = *reinterpret_cast<const f32x4*>(a.gb + c * 4);
 #pragma unroll
-            for (int e = 0; e < 4; e++) v[i][e] = v[i][e] + y[i][e] * rs * gb[e];
-            if (!a.rows_src) *reinterpret_cast<f32x4*>(x + c * 4) = v[i];
+                for (int e = 0; e < 4; e++) v[i][e] = v[i][e] + y[i][e] * rs * gb[e];
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; e++) v[i][e] = v[i][e] + y[i][e];
+            }
+            if (a.x0) {
+                const f32x4 u = *reinterpret_cast<const f32x4*>(a.x0 + (size_t)r * a.width + c * 4);
+#pragma unroll
+                for (int e = 0; e < 4; e++) v[i][e] += u[e];
+            }
+            if (!a.rows_src) *reinterpret_cast<f32x4*>(x_new + c * 4) = v[i];
         }
     }
     if (!a.h) return;
@@ -187,7 +202,6 @@ __global__ __launch_bounds__(256) void norm_rows_vec_kernel(RowArgs a) {
 template <typename ET>
 int norm_rows(const RowArgs& a, hipStream_t st) {
     FX_REQUIRE(a.x && a.rows > 0 && a.width > 0 && a.width <= 16384 && (!a.h || (a.g && a.ldh >= a.width)), "norm_rows: rows=%d width=%d", a.rows, a.width);
-    FX_REQUIRE(!(a.y || a.ys) || a.gb, "norm_rows: no weight for the norm after the sublayer");
     const bool vec = a.width % 4 == 0 && a.ldy % 4 == 0 && a.ldh % 4 == 0;
     if (vec && a.width <= 1024) norm_rows_vec_kernel<ET, 1><<<a.rows, 256, 0, st>>>(a);
     else if (vec && a.width <= 2048) norm_rows_vec_kernel<ET, 2><<<a.rows, 256, 0, st>>>(a);

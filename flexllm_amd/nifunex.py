@@ -2,18 +2,10 @@
 layer's cached rows) or gated linear attention, each with a dense or a mixture feed-forward, norms before and after every
 sublayer.  Reads config.json and the tensor names of a checkpoint; the layers themselves are hybrid.HybridModel's."""
 import math
-import os
-
-import numpy as np
 
 from . import loader, synth
-from .device import to_device
-from .hybrid import HybridModel, MIX_LATENT, MIX_GLA, FF_NONE, FF_DENSE, FF_MOE
+from .hybrid import (ConfigError, HybridModel, check_shapes, dense_shapes, group_weights, upload, MIX_LATENT, MIX_GLA, FF_NONE, FF_DENSE, FF_MOE)
 from .registry import register
-
-
-class ConfigError(ValueError):
-    pass
 
 
 def layer_descriptor(i, layer, shape):
@@ -55,11 +47,6 @@ def tensor_shapes(cfg, a_rank=16):
     """{tensor name: shape} of a checkpoint of this configuration; a_rank: rank of the decay projection, which the
     configuration leaves to the tensors."""
     W, out = cfg["width"], {"embed": (cfg["vocab"], cfg["width"]), "final.norm": (cfg["width"],), "head": (cfg["vocab"], cfg["width"])}
-
-    def feed_forward(pre, ff):
-        out[pre + "gate"] = out[pre + "up"] = (ff, W)
-        out[pre + "down"] = (W, ff)
-
     for i, ly in enumerate(cfg["layers"]):
         mx, mlp, pre = ly["mixer"], ly.get("mlp"), "l%d." % i
         for n in ("norm1", "norm1b") + (("norm2", "norm2b") if mlp else ()):
@@ -78,36 +65,14 @@ def tensor_shapes(cfg, a_rank=16):
             continue
         f = pre + "mlp."
         if mlp["kind"] == "dense":
-            feed_forward(f, mlp["ff"])
+            dense_shapes(out, f, mlp["ff"], W)
         else:
             for e in range(mlp["router"]["experts"]):
-                feed_forward("%se%d." % (f, e), mlp["expert"]["ff"])
+                dense_shapes(out, "%se%d." % (f, e), mlp["expert"]["ff"], W)
             out[f + "router"] = (mlp["router"]["experts"], W)
             if mlp.get("shared"):
-                feed_forward(f + "shared.", mlp["shared"]["ff"])
+                dense_shapes(out, f + "shared.", mlp["shared"]["ff"], W)
                 out[f + "shared.sg"] = (1, W)
-    return out
-
-
-# field of HybridLayerWeights -> tensor name behind 'l<i>.'
-_NORMS = dict(norm1="norm1", norm1b="norm1b", norm2="norm2", norm2b="norm2b")
-_MIX = dict(q="q", o="o", dkv="dkv", dkv_norm="dkv.norm", uk="uk", uv="uv", k="k", v="v", g="g", a1="a1", a2="a2", a2_bias="a2.b", head_norm="norm")
-_MLP = dict(gate="gate", up="up", down="down", router="router", shared_gate="shared.gate", shared_up="shared.up",
-            shared_down="shared.down", shared_sg="shared.sg")
-
-
-def group_weights(cfg, tensor, names):
-    """The weights structure of HybridModel; tensor(name) gives a device array, names the tensors that there are."""
-    out = {"embed": tensor("embed"), "final_norm": tensor("final.norm"), "head": tensor("head"), "layers": []}
-    for i, ly in enumerate(cfg["layers"]):
-        w = {}
-        for table, pre in ((_NORMS, "l%d." % i), (_MIX, "l%d.mix." % i), (_MLP, "l%d.mlp." % i)):
-            w.update({f: tensor(pre + n) for f, n in table.items() if pre + n in names})
-        mlp = ly.get("mlp")
-        if mlp and mlp["kind"] == "moe":
-            for part in ("gate", "up", "down"):
-                w["expert_" + part] = [tensor("l%d.mlp.e%d.%s" % (i, e, part)) for e in range(mlp["router"]["experts"])]
-        out["layers"].append(w)
     return out
 
 
@@ -117,29 +82,20 @@ class Nifunex(HybridModel):
         """weights: group_weights' structure; shapes: {tensor name: shape}."""
         self.cfg = cfg
         layers = [layer_descriptor(i, ly, shapes.__getitem__) for i, ly in enumerate(cfg["layers"])]
-        super().__init__(cfg["width"], cfg["vocab"], cfg["norm"]["eps"], layers, weights, dtype=dtype, max_pos=max_pos, slots=slots)
+        super().__init__(cfg["width"], cfg["vocab"], cfg["norm"]["eps"], layers, weights, dtype=dtype, max_pos=max_pos, slots=slots,
+                         norm_add=1.0, post_norms=True)
 
     @classmethod
     def from_tensors(cls, cfg, tensors, **kw):
         """tensors: {name: host array}, bfloat16 as uint16 bit patterns or any float array (rounded to bfloat16)."""
         want = tensor_shapes(cfg)
-        for name, shape in want.items():
-            if name not in tensors:
-                raise loader.ParameterError("missing tensor %s" % name)
-            got = tuple(tensors[name].shape)
-            free = (0,) if name.endswith(".mix.a1") else (1,) if name.endswith(".mix.a2") else ()
-            if len(got) != len(shape) or any(g != s for k, (g, s) in enumerate(zip(got, shape)) if k not in free):
-                raise loader.ParameterError("%s has shape %s, the configuration says %s" % (name, list(got), list(shape)))
+        check_shapes(tensors, want, lambda name: (0,) if name.endswith(".mix.a1") else (1,) if name.endswith(".mix.a2") else ())
         for i in range(len(cfg["layers"])):
             m = "l%d.mix." % i
             if m + "a1" in want and tensors[m + "a1"].shape[0] != tensors[m + "a2"].shape[1]:
                 raise loader.ParameterError("%sa1 and %sa2 disagree about the rank" % (m, m))
-        dev = {n: to_device(t if t.dtype == np.uint16 else loader.to_bf16(t)) for n, t in tensors.items() if n in want}
+        dev = upload(tensors, want)
         return cls(cfg, group_weights(cfg, dev.__getitem__, dev), {n: tuple(t.shape) for n, t in tensors.items()}, **kw)
-
-    @classmethod
-    def from_dir(cls, path, cfg, **kw):
-        return cls.from_tensors(cfg, loader.read_safetensors(os.path.join(path, "model.safetensors")), **kw)
 
     @classmethod
     def synthetic(cls, cfg, seed=1, a_rank=16, **kw):

@@ -10,7 +10,7 @@ import os
 from ._lib import ensure
 
 # design -> module that registers it on import, the part of the library it needs
-_MODULES = {"Nifunex": ("nifunex", "hybrid")}
+_MODULES = {"Lopazen": ("lopazen", "hybrid"), "Nifunex": ("nifunex", "hybrid")}
 _CLASSES = {}
 
 

@@ -493,10 +493,10 @@ int flexllm_hmt_retrieve(const float* q, const float* kmem, const float* mmem, f
 int flexllm_hmt_stage_input(const float* emb, const float* t_embed, const float* p_buf, float* x_out, int stage, int seq_off,
                             int cur_len, int cur_sum_len, int rec_len, int tail_p, int rows, int hidden, void* stream);
 
-/* ---- floating-point decoder models: layers of latent attention and gated linear attention -------------------------
+/* ---- floating-point decoder models -----------------------------------------------------------------------------------
  * A decoder whose layers are chosen one by one (no counterpart in the reference, which has one quantised graph): each
- * layer is a mixer and a feed-forward, both with an RMS norm before and after (weights stored around zero:
- * rms(x) * (1 + w)) and a float32 residual.  dtype 0: weights, activations between kernels and cached rows in bfloat16
+ * layer is a mixer and a feed-forward, both with an RMS norm before (and, if the design has them, after) and a float32
+ * residual.  dtype 0: weights, activations between kernels and cached rows in bfloat16
  * with float32 sums; dtype 1: everything in float32.  Norms, scores and softmax, routers, the residual and every state
  * are float32 in both.  Weight pointers are device bfloat16 arrays, row-major [out][in], copied and repacked by create.
  *
@@ -506,22 +506,39 @@ int flexllm_hmt_stage_input(const float* emb, const float* t_embed, const float*
  *                       `window` positions are seen, 0: all.  kv_from >= 0: the layer reads the rows of that earlier
  *                       layer and has no dkv of its own.  Rotation: neighbouring pairs, base rot_base, with yarn != 0
  *                       the frequencies are interpolated between f and f / yarn_factor.
+ *   FLEXLLM_MIX_SHARED_KV  attention of `heads` query heads on kv_heads key/value heads (head h uses h / (heads / kv_heads))
+ *                       whose values are the projected keys: W_q h + b_q and W_k h + b_k (no biases when the pointers are
+ *                       null); query and key are RMS-normed per head with weights q_norm and k_norm [dim], the value is
+ *                       the key ahead of its norm (vdim == dim).  No rotation; the query is multiplied by
+ *                       1 + temp_coef * ln(floor((p + 1) / temp_every) + 1) at position p.  sink != 0: one is added to the
+ *                       softmax denominator.  Every earlier position is seen.
  *   FLEXLLM_MIX_GLA     gated linear attention, decay per key channel sigmoid(W_a2 W_a1 h + b)^(1/tau), float32 state
  * Feed-forwards
- *   FLEXLLM_FF_NONE, FLEXLLM_FF_DENSE (clamped gated unit g sigmoid(1.702 g)(u + 1), g = min(gate, limit),
- *   u = clamp(up, -limit, limit)), FLEXLLM_FF_MOE (`top` of `experts` by softmax, weights divided by their sum; an
- *   optional shared expert times sigmoid(W_sg h))
+ *   FLEXLLM_FF_NONE, FLEXLLM_FF_DENSE, FLEXLLM_FF_MOE (`top` of `experts` by softmax, weights divided by their sum; an
+ *   optional shared expert times sigmoid(W_sg h)).  Gated unit `glu`: FLEXLLM_GLU_CLAMPED g sigmoid(1.702 g)(u + 1) with
+ *   g = min(gate, limit), u = clamp(up, -limit, limit); FLEXLLM_GLU_GELU gelu(gate) up, gelu in its tanh form
+ * Around the layers
+ *   Embedding rows are multiplied by embed_scale; `head` may be the embedding matrix itself (same pointer).  The norms'
+ *   effective weights are norm_add + the stored ones, for norm1, norm2, norm1b, norm2b and final_norm.  With post_norms
+ *   a sublayer's output is normed (norm1b, norm2b) before it is added.  Layers loop_start .. loop_stop-1 run loop_times
+ *   times in a row (loop_times 1: no loop), each pass with rows and states of its own; ahead of every pass but the first
+ *   the embedding output is added to the residual.
  *
  * Sequences live in slots: a slot holds the cached rows, the states and the length of one sequence.  reset starts it
  * afresh (nothing of the previous sequence is read again).  One object is used from one stream at a time. */
 #define FLEXLLM_MIX_LATENT 0
 #define FLEXLLM_MIX_GLA 1
+#define FLEXLLM_MIX_SHARED_KV 2
 #define FLEXLLM_FF_NONE 0
 #define FLEXLLM_FF_DENSE 1
 #define FLEXLLM_FF_MOE 2
+#define FLEXLLM_GLU_CLAMPED 0
+#define FLEXLLM_GLU_GELU 1
 typedef struct {
     int layers, width, vocab, max_pos, slots, dtype;
     float eps;
+    float embed_scale, norm_add;
+    int post_norms, loop_start, loop_stop, loop_times;
 } flexllm_hybrid_config;
 typedef struct {
     int mixer, heads, dim, vdim;
@@ -531,6 +548,9 @@ typedef struct {
     double rot_base, yarn_factor, yarn_original, yarn_fast, yarn_slow;
     int a_rank;                                 /* gated linear attention */
     float tau;
+    int kv_heads, sink, temp_every;             /* attention whose values are its keys */
+    float temp_coef;
+    int glu;
     int ff_kind, ff, experts, top, shared_ff;   /* ff: of the dense layer or of an expert; shared_ff 0: none */
     float limit, shared_limit;
 } flexllm_hybrid_layer;
@@ -538,7 +558,8 @@ typedef struct {
     const uint16_t *norm1, *norm1b, *norm2, *norm2b;                       /* [width] */
     const uint16_t *q, *o;                                                 /* both mixers */
     const uint16_t *dkv, *dkv_norm, *uk, *uv;                              /* latent attention */
-    const uint16_t *k, *v, *g, *a1, *a2, *a2_bias, *head_norm;             /* gated linear attention */
+    const uint16_t *k, *v, *g, *a1, *a2, *a2_bias, *head_norm;             /* gated linear attention (k: shared key/value attention too) */
+    const uint16_t *q_bias, *k_bias, *q_norm, *k_norm;                     /* shared key/value attention */
     const uint16_t *gate, *up, *down;                                      /* dense */
     const uint16_t *router, *shared_gate, *shared_up, *shared_down, *shared_sg;
     const uint16_t *const *expert_gate, *const *expert_up, *const *expert_down;   /* host arrays of `experts` device pointers */
@@ -556,7 +577,7 @@ int flexllm_hybrid_reset(flexllm_hybrid* m, int slot, void* stream);
 int flexllm_hybrid_length(const flexllm_hybrid* m, int slot, int* length);
 /* Run n further tokens (device ids) of the slot's sequence from what its cache and states hold.  want (host, ascending
  * places in 0..n-1) names the n_want tokens whose logits are written to logits (device [n_want][vocab]).  layers_out
- * (device [layers][n][width] or NULL) receives the residual after every layer. */
+ * (device [layer runs][n][width] or NULL; a looped layer counts once per pass) receives the residual after every layer. */
 int flexllm_hybrid_step(flexllm_hybrid* m, int slot, const int* tokens, int n, const int* want, int n_want, float* logits,
                         float* layers_out, void* stream);
 /* `steps` tokens from *token_io (device; fed first, the last drawn token on return) into tokens_out (device [steps]):
