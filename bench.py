@@ -326,7 +326,7 @@ def module_legs(fx, lib, synth, ops, stream, Event, peaks=None):
     return out
 
 
-# ---- Nifunex: layers of real models' sizes, random weights ------------------------------------------------------------
+# ---- Nifunex and Lopazen: layers of real models' sizes, random weights ------------------------------------------------
 BF16_PEAK_TFLOPS = 2500.0      # MI355X published dense bf16 MFMA rate
 
 
@@ -347,6 +347,30 @@ def nifunex_config(name):
         else:
             out.append({"type": "gla", "mixer": {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0}, "mlp": mlp})
     return {"architecture": "Nifunex", "width": width, "vocab": vocab, "norm": {"eps": 1e-6}, "layers": out}
+
+
+def lopazen_config(name):
+    """Sizes for --lopazen.  1b has the layer sizes, layer count and vocabulary of Llama-3.2-1B; 1b-loop runs the same sixteen
+    layers' worth from ten layers, six of them twice; 8b has the layer sizes of published 8B models."""
+    heads, kv_heads, dim, width, ff, layers, loop = {"1b": (32, 8, 64, 2048, 8192, 16, (0, 0, 1)), "1b-loop": (32, 8, 64, 2048, 8192, 10, (2, 8, 2)),
+                                                     "8b": (32, 8, 128, 4096, 14336, 4, (0, 0, 1))}[name]
+    ly = {"type": "attention", "mlp": {"kind": "dense", "ff": ff},
+          "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "q_temp": {"coef": 0.1, "every": 1024}}}
+    return {"architecture": "Lopazen", "width": width, "vocab": 128256, "norm": {"eps": 1e-6}, "embedding": {"scale": width ** 0.5},
+            "layers": [ly] * layers, "loop": dict(zip(("start", "stop", "times"), loop))}
+
+
+def lopazen_work(cfg, shapes, tokens, context):
+    """As nifunex_work; a looped layer's weights and rows are read, and its products formed, once per pass."""
+    size = lambda n: int(np.prod(shapes[n]))
+    by, ops = 2 * size("embed"), 0
+    for i, ly in enumerate(cfg["layers"]):
+        mx = ly["mixer"]
+        mats = sum(size(n) for n in shapes if n.startswith("l%d." % i) and len(shapes[n]) == 2)
+        passes = cfg["loop"]["times"] if cfg["loop"]["start"] <= i < cfg["loop"]["stop"] else 1
+        by += passes * (2 * mats + mx["kv_heads"] * context * (2 * mx["dim"] + 4))
+        ops += passes * (2 * tokens * mats + 2 * tokens * (tokens + 1) * mx["heads"] * mx["dim"])
+    return by, ops
 
 
 def nifunex_work(cfg, shapes, tokens, context):
@@ -374,17 +398,18 @@ def nifunex_work(cfg, shapes, tokens, context):
     return by + 2 * size("head"), ops
 
 
-def nifunex_leg(name, steps, warmup, prompts=(1024, 4096), seed=3):
+def hybrid_leg(design, name, steps, warmup, prompts=(1024, 4096), seed=3):
+    import importlib
     import flexllm_amd as fx
-    from flexllm_amd import synth
     from flexllm_amd.device import Event, device_sync
-    from flexllm_amd.nifunex import Nifunex, tensor_shapes
-    cfg = nifunex_config(name)
-    shapes = tensor_shapes(cfg)
-    m = Nifunex.synthetic(cfg, seed=seed, max_pos=max(prompts) + warmup + steps + 8)
+    from flexllm_amd.registry import model_class
+    config, work = {"Nifunex": (nifunex_config, nifunex_work), "Lopazen": (lopazen_config, lopazen_work)}[design]
+    cfg, cls = config(name), model_class(design)
+    shapes = importlib.import_module(cls.__module__).tensor_shapes(cfg)
+    m = cls.synthetic(cfg, seed=seed, max_pos=max(prompts) + warmup + steps + 8)
     st = m.stream()
     toks = fx.to_device(np.random.default_rng(7).integers(0, cfg["vocab"], max(prompts)).astype(np.int32))
-    out = {"config": {"width": cfg["width"], "layers": len(cfg["layers"]), "vocab": cfg["vocab"], "mlp": cfg["layers"][0]["mlp"]}, "prefill": {}}
+    out = {"config": {"width": cfg["width"], "layers": len(cfg["layers"]), "layer_runs": m.layer_runs, "vocab": cfg["vocab"], "mlp": cfg["layers"][0]["mlp"]}, "prefill": {}}
 
     def prompt(n):
         slot = m.pool.acquire("p")
@@ -393,7 +418,7 @@ def nifunex_leg(name, steps, warmup, prompts=(1024, 4096), seed=3):
 
     for n in prompts:
         us = _time(st, Event, lambda i: prompt(n), 5)
-        _, ops = nifunex_work(cfg, shapes, n, n)
+        _, ops = work(cfg, shapes, n, n)
         out["prefill"][str(n)] = {"ms": round(us / 1e3, 3), "tokens_per_s": round(n / us * 1e6, 1), "TFLOPs": round(ops / us / 1e6, 1),
                                   "mfma_frac": round(ops / us / 1e6 / BF16_PEAK_TFLOPS, 4)}
     slot = m.pool.acquire("d")
@@ -410,21 +435,21 @@ def nifunex_leg(name, steps, warmup, prompts=(1024, 4096), seed=3):
     device_sync()
     m.check()
     us = e0.elapsed_ms(e1) * 1e3 / steps
-    by, _ = nifunex_work(cfg, shapes, 1, max(prompts))
+    by, _ = work(cfg, shapes, 1, max(prompts))
     out["decode"] = {"context": max(prompts), "us_per_token": round(us, 2), "tokens_per_s": round(1e6 / us, 1), "bytes_per_token": by,
                      "GBs": round(by / us / 1e3, 1), "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4), "distinct_tokens": len(set(gen.numpy()[:steps].tolist()))}
     m.close()
     return out
 
 
-def nifunex_main(args):
-    """--nifunex: decode and prefill of the Nifunex sizes beside Llama-3.2-1B W8A8 in the same process.  One JSON line."""
+def hybrid_main(args, design, names, prompts):
+    """--nifunex, --lopazen: decode and prefill of a design's sizes beside Llama-3.2-1B W8A8 in the same process.  One JSON line."""
     import flexllm_amd as fx
     from flexllm_amd import llama, synth
     from flexllm_amd.device import Event
-    res = {"metric": "Nifunex decode tok/s + prefill ms", "dtype": "bf16", "data": "synthetic", "device": fx.device.device_name(), "sizes": {}}
-    for name in args.nifunex.split(","):
-        res["sizes"][name] = nifunex_leg(name, args.steps, args.warmup, tuple(int(n) for n in args.nifunex_prompts.split(",")))
+    res = {"metric": design + " decode tok/s + prefill ms", "dtype": "bf16", "data": "synthetic", "device": fx.device.device_name(), "sizes": {}}
+    for name in names.split(","):
+        res["sizes"][name] = hybrid_leg(design, name, args.steps, args.warmup, tuple(int(n) for n in prompts.split(",")))
     if not args.no_prefill:
         cfg = llama.make_config()
         model = llama.Llama(cfg, llama.synth_weights(cfg, seed=1, device=True, embed_range=0.03))
@@ -469,6 +494,9 @@ def main():
                     help="only run the Nifunex sizes (1b-dense, 1b-moe, 8b-dense; all when none is named) and, unless --no-prefill, "
                          "Llama-3.2-1B W8A8 beside them")
     ap.add_argument("--nifunex-prompts", default="1024,4096", help="prompt lengths of the --nifunex legs; decoding starts behind the longest")
+    ap.add_argument("--lopazen", nargs="?", const="1b,1b-loop,8b", default=None, metavar="SIZES",
+                    help="the same for the Lopazen sizes (1b, 1b-loop, 8b)")
+    ap.add_argument("--lopazen-prompts", default="1024,4096", help="prompt lengths of the --lopazen legs")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on one GPU only (no collectives, no sharding); use --gpus 1", file=sys.stderr)
@@ -479,9 +507,10 @@ def main():
     from flexllm_amd.device import Event, device_sync
 
     lib = fx.lib()
-    if args.nifunex:
-        nifunex_main(args)
-        return
+    for design, names, prompts in (("Nifunex", args.nifunex, args.nifunex_prompts), ("Lopazen", args.lopazen, args.lopazen_prompts)):
+        if names:
+            hybrid_main(args, design, names, prompts)
+            return
     if args.copy_probe:
         n = 1 << 30
         src = synth.device_i8((n,), 1)

@@ -386,11 +386,11 @@ using namespace fx;
 
 extern "C" {
 
-int flexllm_linear_float_gemm(const void* a, const void* w, void* y, float* y32, int m, int k, int n, int n_split, int glu, float limit,
+int flexllm_linear_float_gemm(const void* a, const void* w, const float* bias, void* y, float* y32, int m, int k, int n, int n_split, int glu, float limit,
                               int dtype, void* stream) {
-    FX_REQUIRE(dtype == 0 || dtype == 1, "linear_float_gemm: dtype=%d", dtype);
+    FX_REQUIRE((dtype == 0 || dtype == 1) && glu >= 0 && glu <= 1 + FLEXLLM_GLU_GELU, "linear_float_gemm: dtype=%d glu=%d", dtype, glu);
     GemmArgs g;
-    g.a = a; g.w = w; g.lda = k; g.m = m; g.n = n; g.k = k; g.n_split = n_split; g.glu = glu; g.limit = limit;
+    g.a = a; g.w = w; g.lda = k; g.m = m; g.n = n; g.k = k; g.n_split = n_split; g.glu = glu; g.limit = limit; g.bias = bias;
     g.y = y; g.ldy = glu ? n_split / 2 : n_split; g.y32 = y32; g.ldy32 = n - n_split;
     return dtype == 0 ? gemm_float<bf16_t>(g, as_stream(stream)) : gemm_float<float>(g, as_stream(stream));
 }

@@ -421,15 +421,15 @@ def sample_topk_f32(logits, top_k=5, rand=0.5, enable_sub_max=True, stream=None)
     return int(tok.numpy()[0]), idx.numpy(), val.numpy(), prob.numpy()
 
 
-def linear_float(a, w, n_split=None, glu=False, limit=0.0, stream=None):
+def linear_float(a, w, n_split=None, glu=0, limit=0.0, bias=None, stream=None):
     """(columns below n_split in the element type, the others in float32) of a w^T; a [m][k], w [n][k] device arrays,
-    uint16 (bfloat16) or float32, k a multiple of 64.  glu: the first part is the clamped gated unit of interleaved
-    gate / up rows."""
+    uint16 (bfloat16) or float32, k a multiple of 64.  glu 1 (clamped), 2 (gelu): the first part is the gated unit of
+    interleaved gate / up rows.  bias: float32 [n]."""
     m, k = a.shape
     n = w.shape[0]
     n_split = n if n_split is None else n_split
     y = DeviceArray((m, n_split // 2 if glu else n_split), a.dtype) if n_split else None
     y32 = DeviceArray((m, n - n_split), np.float32) if n_split < n else None
-    check(lib().flexllm_linear_float_gemm(_p(a), _p(w), _p(y), _p(y32), m, k, n, n_split, int(glu), C.c_float(limit),
+    check(lib().flexllm_linear_float_gemm(_p(a), _p(w), _p(bias), _p(y), _p(y32), m, k, n, n_split, int(glu), C.c_float(limit),
                                           int(a.dtype == np.float32), _s(stream)))
     return y, y32

@@ -592,8 +592,9 @@ int flexllm_hybrid_generate(flexllm_hybrid* m, int slot, const int* prompt, int 
 int flexllm_hybrid_check(flexllm_hybrid* m);
 /* The GEMM behind the prompt path on its own: a [m][k], w [n][k] of the element type (dtype as in the configuration),
  * k % 64 == 0.  Columns below n_split go to y (element type, [m][n_split], or with glu [m][n_split/2]: rows 2i / 2i+1 of w
- * are gate and up of unit i), the others to y32 (float32 [m][n - n_split]); n_split must keep pairs together. */
-int flexllm_linear_float_gemm(const void* a, const void* w, void* y, float* y32, int m, int k, int n, int n_split, int glu, float limit,
+ * are gate and up of unit i), the others to y32 (float32 [m][n - n_split]); n_split must keep pairs together.
+ * bias [n] or NULL is added first; glu: 0, or 1 + FLEXLLM_GLU_*. */
+int flexllm_linear_float_gemm(const void* a, const void* w, const float* bias, void* y, float* y32, int m, int k, int n, int n_split, int glu, float limit,
                               int dtype, void* stream);
 int flexllm_rt_fill_uniform_bf16(uint16_t* dst, size_t n, uint64_t seed, float lo, float hi, void* stream);
 
