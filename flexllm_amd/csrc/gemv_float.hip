@@ -245,8 +245,9 @@ __global__ __launch_bounds__(256) void gemv_float_kernel(GemvArgs g) {
 
 template <typename ET, int R, int S>
 static int launch_gemv_rs(const GemvArgs& g, int pro, int rows_y, hipStream_t st) {
-    // workgroups that share the chip at a time; each walks its groups with the next one's weights in flight
-    int wgs = 1024 / rows_y;
+    // workgroups that share the chip at a time (two per CU where the vector takes a third of LDS or more); each walks its
+    // groups with the next one's weights in flight
+    int wgs = (S > 4 ? 512 : 1024) / rows_y;
     if (wgs < 128) wgs = 128;
     const int ng = (g.n + R - 1) / R;
     const dim3 grid(ng < wgs ? ng : wgs, rows_y);
@@ -258,8 +259,10 @@ static int launch_gemv_rs(const GemvArgs& g, int pro, int rows_y, hipStream_t st
         else gemv_float_kernel<ET, R, S, PRO, false><<<grid, 256, lds, st>>>(g);                   \
     } while (0)
     if (pro == 0) FX_GEMV(0);
-    else if (pro == 1) FX_GEMV(1);
-    else FX_GEMV(2);
+    if constexpr (S <= 4) {                               // longer rows: gemv_float asks for the plain linear only
+        if (pro == 1) FX_GEMV(1);
+        if (pro == 2) FX_GEMV(2);
+    }
 #undef FX_GEMV
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
@@ -278,6 +281,7 @@ int gemv_float(const GemvArgs& g, int pro, int tokens, hipStream_t st) {
         return launch_gemv_rs<ET, 4, 1>(g, pro, rows_y, st);
     }
     if (steps == 2) return launch_gemv_rs<ET, 4, 2>(g, pro, rows_y, st);
+    if (steps > 4 && pro == 0) return launch_gemv_rs<ET, 2, 8>(g, pro, rows_y, st);
     return launch_gemv_rs<ET, 2, 4>(g, pro, rows_y, st);
 }
 template int gemv_float<bf16_t>(const GemvArgs&, int, int, hipStream_t);
