@@ -35,39 +35,41 @@ __device__ __forceinline__ float group_sum(float v) {
     return v;
 }
 
-// ---- rows of a step into the cache: one wave per row --------------------------------------------------------------
-template <typename ET>
+// ---- rows of a step into the cache: LPR lanes per row -------------------------------------------------------------
+template <typename ET, int LPR>
 __global__ __launch_bounds__(256) void shared_kv_store_kernel(SharedKvDims d, const float* __restrict__ k, int ldk, SharedKvRows<ET> c,
                                                               const int* __restrict__ state, int total) {
-    const int idx = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (idx >= total) return;
+    const int n = blockIdx.x * (256 / LPR) + threadIdx.x / LPR, lane = threadIdx.x % LPR, idx = min(n, total - 1);
     const int tok = idx / d.kv_heads, g = idx - tok * d.kv_heads, pos = state[0] + tok;
-    if (pos >= d.capacity) return;
+    const bool mine = n < total && pos < d.capacity;
     const float* x = k + (size_t)tok * ldk + g * d.dimp;
-    ET* row = c.row + ((size_t)g * d.capacity + pos) * d.dimp;
+    const size_t at = (size_t)g * d.capacity + pos;
     float ss = 0.0f;
-    for (int i = lane * 4; i < d.dimp; i += 256) {
+    for (int i = lane * 4; i < d.dimp; i += LPR * 4) {
         const f32x4 v = *reinterpret_cast<const f32x4*>(x + i);
 #pragma unroll
         for (int e = 0; e < 4; e++) ss = fma_f(v[e], v[e], ss);
+        if (!mine) continue;
         if constexpr (std::is_same<ET, float>::value) {
-            *reinterpret_cast<f32x4*>(row + i) = v;
+            *reinterpret_cast<f32x4*>(c.row + at * d.dimp + i) = v;
         } else {
             bf16x4 b;
 #pragma unroll
             for (int e = 0; e < 4; e++) b[e] = (bf16_t)v[e];
-            *reinterpret_cast<bf16x4*>(row + i) = b;
+            *reinterpret_cast<bf16x4*>(c.row + at * d.dimp + i) = b;
         }
     }
-    ss = wave_sum(ss);
-    if (lane == 0) c.inv_rms[(size_t)g * d.capacity + pos] = 1.0f / sqrtf(ss / (float)d.dim + d.eps);
+    ss = group_sum<LPR>(ss);
+    if (lane == 0 && mine) c.inv_rms[at] = 1.0f / sqrtf(ss / (float)d.dim + d.eps);
 }
 
 template <typename ET>
 int shared_kv_store(const SharedKvDims& d, const float* k, int ldk, SharedKvRows<ET> c, const int* state, int tokens, hipStream_t st) {
     FX_REQUIRE(k && c.row && c.inv_rms && state && tokens > 0 && ldk >= d.kv_heads * d.dimp && ldk % 4 == 0, "shared_kv_store: tokens=%d ldk=%d", tokens, ldk);
     const int total = tokens * d.kv_heads;
-    shared_kv_store_kernel<ET><<<(total + 3) / 4, 256, 0, st>>>(d, k, ldk, c, state, total);
+    if (d.dimp <= 64) shared_kv_store_kernel<ET, 16><<<(total + 15) / 16, 256, 0, st>>>(d, k, ldk, c, state, total);
+    else if (d.dimp <= 128) shared_kv_store_kernel<ET, 32><<<(total + 7) / 8, 256, 0, st>>>(d, k, ldk, c, state, total);
+    else shared_kv_store_kernel<ET, 64><<<(total + 3) / 4, 256, 0, st>>>(d, k, ldk, c, state, total);
     FX_LAUNCH_CHECK();
     return FLEXLLM_OK;
 }
